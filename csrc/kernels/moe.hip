@@ -5,7 +5,9 @@
 //   * alignment: the (token, choice) pairs sorted by expert (counting sort in one workgroup),
 //   * grouped GEMMs over the sorted rows: gate | up with the SiLU unit fused, then down, written back in (token,
 //     choice) order,
-//   * boundary: x += mixer + shared * gate + sum_k weight_k expert_k in fp32, then the next RMS norm, one pass.
+//   * boundary: x += mixer + shared * gate + sum_k weight_k expert_k in fp32, then the next RMS norm, one pass;
+//   * post-norm boundary: the sublayer's output is RMS-normed before it joins x (and two side-by-side mixers' outputs
+//     are normed apiece before they are added), one pass too.
 // Activations are bf16 or fp32 (dt: 0 = bf16, 1 = fp32); logits, scores, weights and the residual are fp32 in both.
 #include "common.h"
 
@@ -29,9 +31,16 @@ constexpr int RT_MAXTOP = 16;
 
 // One token's choice from its logits z [R] (overwritten): scores = softmax of the first E; the `keep` best groups
 // (a group's score is its best expert's) are open; the best `top` experts of the open groups, by falling score, ties
-// to the lower index, weighted by their scores as they are; row E (if any) is the shared expert's gate logit.
+// to the lower index, weighted by their scores as they are; row E (if any) is the shared expert's gate logit.  With
+// `corr` [E] the choice goes by score + corr (the weights do not).  The last nid of the E rows are identity experts:
+// their weights are summed into idw[t], and the choice's own weight becomes 0 (there is no expert output to weigh).
+struct RouteExtra {
+  const float* corr;
+  int nid;
+  float* idw;
+};
 __device__ void route_select(float* z, int E, int R, int top, int ngroups, int keep, int t, int* __restrict__ ids,
-                             float* __restrict__ wts, float* __restrict__ sgate) {
+                             float* __restrict__ wts, float* __restrict__ sgate, const RouteExtra& rx) {
   if (R > E && sgate != nullptr) sgate[t] = 1.f / (1.f + expf(-z[E]));
   float mx = -INFINITY;
   for (int e = 0; e < E; ++e) mx = fmaxf(mx, z[e]);
@@ -65,13 +74,14 @@ __device__ void route_select(float* z, int E, int R, int top, int ngroups, int k
     else open_3 |= bit;
   }
   // the best `top` experts of the open groups; a taken expert's logit is overwritten with -inf
+  float idsum = 0.f;
   for (int n = 0; n < top; ++n) {
     int be = -1;
     float bv = -INFINITY;
     for (int e = 0; e < E; ++e) {
-      if (!is_open(e / per)) continue;
-      const float v = z[e];
-      if (v > bv || (be < 0 && v > -INFINITY)) {
+      if (!is_open(e / per) || z[e] == -INFINITY) continue;
+      const float v = rx.corr ? fmaf(expf(z[e] - mx), inv, rx.corr[e]) : z[e];
+      if (v > bv || be < 0) {
         be = e;
         bv = v;
       }
@@ -82,9 +92,13 @@ __device__ void route_select(float* z, int E, int R, int top, int ngroups, int k
       continue;
     }
     ids[(size_t)t * top + n] = be;
-    wts[(size_t)t * top + n] = expf(bv - mx) * inv;
+    const float wt = expf(z[be] - mx) * inv;
+    const bool ident = be >= E - rx.nid;
+    wts[(size_t)t * top + n] = ident ? 0.f : wt;
+    if (ident) idsum += wt;
     z[be] = -INFINITY;
   }
+  if (rx.idw != nullptr) rx.idw[t] = idsum;
 }
 
 // h [T][ld] (the normed layer input); wr [R][W] fp32, rows 0 .. E-1 the experts, row E (R = E + 1) the shared expert's
@@ -95,7 +109,7 @@ template <typename T>
 __global__ void __launch_bounds__(256)
 moe_route_kernel(const T* __restrict__ h, int ld, const float* __restrict__ wr, int W, int E, int R, int top,
                  int ngroups, int keep, int* __restrict__ ids, float* __restrict__ wts, float* __restrict__ sgate,
-                 int T_, int vec) {
+                 int T_, int vec, RouteExtra rx) {
   extern __shared__ __attribute__((aligned(16))) float rsm[];
   float* hs = rsm;                   // [RT_TOK][RT_LD]
   float* ws = hs + RT_TOK * RT_LD;   // [R][RT_LD]
@@ -121,7 +135,12 @@ moe_route_kernel(const T* __restrict__ h, int ld, const float* __restrict__ wr, 
         for (int i = 0; i < 8; ++i) hv[i] = bits2f(v[i]);
       } else {
 #pragma unroll
-        for (int i = 0; i < 8; ++i) hv[i] = hok ? ldm(h + (size_t)(t0 + tt) * ld + k0 + kv + i) : 0.f;
+        for (int i = 0; i < 8; i += 4) {
+          const f32x4_t v = hok ? *reinterpret_cast<const f32x4_t*>(h + (size_t)(t0 + tt) * ld + k0 + kv + i)
+                                : f32x4_t{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+          for (int j = 0; j < 4; ++j) hv[i + j] = v[j];
+        }
       }
       const int nvec = R * (RT_KC / 4);
       for (int base = 0; base < nvec; base += 256 * 4) {
@@ -176,7 +195,7 @@ moe_route_kernel(const T* __restrict__ h, int ld, const float* __restrict__ wr, 
     if (part + 16 * j < R) lgs[tok * (R + 1) + part + 16 * j] = acc[j];
   __syncthreads();
   if (threadIdx.x >= RT_TOK || t0 + threadIdx.x >= T_) return;
-  route_select(lgs + threadIdx.x * (R + 1), E, R, top, ngroups, keep, t0 + threadIdx.x, ids, wts, sgate);
+  route_select(lgs + threadIdx.x * (R + 1), E, R, top, ngroups, keep, t0 + threadIdx.x, ids, wts, sgate, rx);
 }
 
 // A few tokens (decode rows): one workgroup per token, one wave per logit row (rows w, w + 4, ...), the lanes split the
@@ -186,7 +205,7 @@ template <typename T>
 __global__ void __launch_bounds__(256)
 moe_route_rows_kernel(const T* __restrict__ h, int ld, const float* __restrict__ wr, int W, int E, int R, int top,
                       int ngroups, int keep, int* __restrict__ ids, float* __restrict__ wts,
-                      float* __restrict__ sgate, int vec) {
+                      float* __restrict__ sgate, int vec, RouteExtra rx) {
   __shared__ float z[RT_MAXR + 1];
   const int t = blockIdx.x, lane = threadIdx.x & 63, wid = threadIdx.x >> 6;
   const T* hr = h + (size_t)t * ld;
@@ -202,7 +221,11 @@ moe_route_rows_kernel(const T* __restrict__ h, int ld, const float* __restrict__
           for (int i = 0; i < 8; ++i) hv[i] = bits2f(v[i]);
         } else {
 #pragma unroll
-          for (int i = 0; i < 8; ++i) hv[i] = ldm(hr + k + i);
+          for (int i = 0; i < 8; i += 4) {
+            const f32x4_t v = *reinterpret_cast<const f32x4_t*>(hr + k + i);
+#pragma unroll
+            for (int j = 0; j < 4; ++j) hv[i + j] = v[j];
+          }
         }
         const f32x4_t w0 = *reinterpret_cast<const f32x4_t*>(w + k), w1 = *reinterpret_cast<const f32x4_t*>(w + k + 4);
 #pragma unroll
@@ -217,7 +240,7 @@ moe_route_rows_kernel(const T* __restrict__ h, int ld, const float* __restrict__
     if (lane == 0) z[r] = a;
   }
   __syncthreads();
-  if (threadIdx.x == 0) route_select(z, E, R, top, ngroups, keep, t, ids, wts, sgate);
+  if (threadIdx.x == 0) route_select(z, E, R, top, ngroups, keep, t, ids, wts, sgate, rx);
 }
 
 // ------------------------------------------------------------------------------------------------ alignment
@@ -271,6 +294,7 @@ __global__ void moe_table_route_kernel(const int* __restrict__ tok, const int* _
 // the "experts" are the E heads, `top` holds the token count, row r of the sorted order is token r % top of head
 // r / top, i.e. row (r % top) * E + r / top of a and out -- no offs / order arrays): with `gate`, element (t, h, n) of
 // the result is multiplied by sigmoid(gate[t * gate_ld + h * N + n]).
+// GATED 3: gathered rows as in 1, one branch (w = [E][N][K]), out = max(a . w_n, 0)^2 in sorted order.
 struct MoeEpi {
   float limit, alpha, shift;
   const void* gate;
@@ -281,6 +305,11 @@ __device__ __forceinline__ float glu_unit(float g, float u, const MoeEpi& ep) {
   u = fminf(fmaxf(u, -ep.limit), ep.limit);
   return g / (1.f + expf(-ep.alpha * g)) * (u + ep.shift);
 }
+__device__ __forceinline__ float relu2_unit(float v) {
+  v = fmaxf(v, 0.f);
+  return v * v;
+}
+constexpr bool moe_gathers(int gated) { return gated == 1 || gated == 3; }
 template <int GATED> __device__ __forceinline__ int moe_off(const int* offs, int e, int top) {
   return GATED == 2 ? e * top : offs[e];
 }
@@ -325,7 +354,7 @@ moe_gemm_kernel(const T* __restrict__ a, int lda, const T* __restrict__ w, const
   const int tx = threadIdx.x & 15, ty = threadIdx.x >> 4;
   if (threadIdx.x < MG_M) {
     const int r = r0 + threadIdx.x;
-    rows[threadIdx.x] = r < rend ? (GATED == 1 ? order[r] / top : GATED == 2 ? moe_order<2>(order, r, top, E) : r) : -1;
+    rows[threadIdx.x] = r < rend ? (moe_gathers(GATED) ? order[r] / top : GATED == 2 ? moe_order<2>(order, r, top, E) : r) : -1;
   }
   const size_t wrows = GATED == 1 ? (size_t)2 * N : (size_t)N;
   const T* we = w + (size_t)e * wrows * K;
@@ -367,13 +396,14 @@ moe_gemm_kernel(const T* __restrict__ a, int lda, const T* __restrict__ w, const
   for (int i = 0; i < 2; ++i) {
     const int r = r0 + ty + 16 * i;
     if (r >= rend) continue;
-    const size_t orow = GATED == 1 ? (size_t)r : (size_t)moe_order<GATED>(order, r, top, E);
+    const size_t orow = moe_gathers(GATED) ? (size_t)r : (size_t)moe_order<GATED>(order, r, top, E);
 #pragma unroll
     for (int j = 0; j < 4; ++j) {
       const int n = n0 + tx + 16 * j;
       if (n >= N) continue;
       float v = acc[0][i][j];
       if (GATED == 1) v = glu_unit(v, acc[GATED == 1 ? 1 : 0][i][j], ep);
+      if (GATED == 3) v = relu2_unit(v);
       if (GATED == 2) v *= head_gate_of<GATED, T>(ep, orow, n, E, N);
       stm(out + orow * ldo + n, v);
     }
@@ -409,7 +439,7 @@ moe_gemm_mfma_kernel(const bf16* __restrict__ a, int lda, const bf16* __restrict
   const int wr = (wid >> 1) * 16, wc = (wid & 1) * 32;
   if (threadIdx.x < MG_M) {
     const int r = r0 + threadIdx.x;
-    rows[threadIdx.x] = r < rend ? (GATED == 1 ? order[r] / top : GATED == 2 ? moe_order<2>(order, r, top, E) : r) : -1;
+    rows[threadIdx.x] = r < rend ? (moe_gathers(GATED) ? order[r] / top : GATED == 2 ? moe_order<2>(order, r, top, E) : r) : -1;
   }
   const size_t wrows = GATED == 1 ? (size_t)2 * N : (size_t)N;
   const bf16* we = w + (size_t)e * wrows * K;
@@ -452,13 +482,14 @@ moe_gemm_mfma_kernel(const bf16* __restrict__ a, int lda, const bf16* __restrict
   for (int i = 0; i < 4; ++i) {
     const int r = r0 + wr + 4 * quad + i;
     if (r >= rend) continue;
-    const size_t orow = GATED == 1 ? (size_t)r : (size_t)moe_order<GATED>(order, r, top, E);
+    const size_t orow = moe_gathers(GATED) ? (size_t)r : (size_t)moe_order<GATED>(order, r, top, E);
 #pragma unroll
     for (int c = 0; c < 2; ++c) {
       const int n = n0 + wc + 16 * c + ql;
       if (n >= N) continue;
       float v = acc[0][c][i];
       if (GATED == 1) v = glu_unit(v, acc[GATED == 1 ? 1 : 0][c][i], ep);
+      if (GATED == 3) v = relu2_unit(v);
       if (GATED == 2) v *= head_gate_of<GATED, bf16>(ep, orow, n, E, N);
       out[orow * ldo + n] = (bf16)v;
     }
@@ -494,7 +525,7 @@ moe_gemm_big_kernel(const bf16* __restrict__ a, int lda, const bf16* __restrict_
   const int wr = (wid >> 1) * 64, wc = (wid & 1) * 64;
   if (threadIdx.x < TM) {
     const int r = r0 + threadIdx.x;
-    rows[threadIdx.x] = r < rend ? (GATED == 1 ? order[r] / top : GATED == 2 ? moe_order<2>(order, r, top, E) : r) : -1;
+    rows[threadIdx.x] = r < rend ? (moe_gathers(GATED) ? order[r] / top : GATED == 2 ? moe_order<2>(order, r, top, E) : r) : -1;
   }
   __syncthreads();
   const size_t wrows = GATED == 1 ? (size_t)2 * N : (size_t)N;
@@ -565,13 +596,14 @@ moe_gemm_big_kernel(const bf16* __restrict__ a, int lda, const bf16* __restrict_
     for (int c = 0; c < 4; ++c) {
       const int r = r0 + wr + 16 * i + 4 * quad + c;
       if (r >= rend) continue;
-      const size_t orow = GATED == 1 ? (size_t)r : (size_t)moe_order<GATED>(order, r, top, E);
+      const size_t orow = moe_gathers(GATED) ? (size_t)r : (size_t)moe_order<GATED>(order, r, top, E);
 #pragma unroll
       for (int j = 0; j < 4; ++j) {
         const int n = n0 + wc + 16 * j + ql;
         if (n >= N) continue;
         float v = acc[0][i][j][c];
         if (GATED == 1) v = glu_unit(v, acc[NB - 1][i][j][c], ep);
+        if (GATED == 3) v = relu2_unit(v);
         if (GATED == 2) v *= head_gate_of<GATED, bf16>(ep, orow, n, E, N);
         out[orow * ldo + n] = (bf16)v;
       }
@@ -720,6 +752,149 @@ residual_rmsnorm_vec_kernel(float* __restrict__ x, float keep, const T* __restri
   }
 }
 
+// ------------------------------------------------------------------------------------------------ post-norm boundary
+// x [T][H] fp32, in place.  With unit(v) = v / sqrt(mean(v^2) + eps):
+//   y <- bscale * (unit(a) * wa + unit(b) * wb)            with wa (two mixers side by side; b and wb optional), else
+//   y <- a + sum_k ecoef_(t,k) e_(t,k) + idw_t x           every addend optional; a pair of weight 0 is not read
+//   x <- x + mult * unit(y) * w                            (w null: x stays)
+//   out <- unit(x) * wn, or x itself without wn, in the activation type (out null: nothing)
+// grid (T): a workgroup holds its row in registers, V elements at a time, PN_PER groups per thread.
+constexpr int PN_PER = 4;
+template <typename T, int V> __device__ __forceinline__ void ldv(const T* p, float (&v)[V]) {
+  if (V == 4) {
+    const f32x4_t t = ld4(p);
+#pragma unroll
+    for (int i = 0; i < V; ++i) v[i] = t[i & 3];
+  } else {
+    v[0] = ldm(p);
+  }
+}
+template <typename T, int V> __device__ __forceinline__ void stv(T* p, const float (&v)[V]) {
+  if (V == 4) st4(p, f32x4_t{v[0], v[V > 1 ? 1 : 0], v[V > 2 ? 2 : 0], v[V > 3 ? 3 : 0]});
+  else stm(p, v[0]);
+}
+// the sums of two values over the workgroup; `red` holds 32 floats
+__device__ __forceinline__ void block_sum2(float& a, float& b, float* red) {
+  const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6, nw = blockDim.x >> 6;
+  a = wave_sum(a);
+  b = wave_sum(b);
+  __syncthreads();
+  if (lane == 0) {
+    red[wid] = a;
+    red[16 + wid] = b;
+  }
+  __syncthreads();
+  a = b = 0.f;
+  for (int i = 0; i < nw; ++i) {
+    a += red[i];
+    b += red[16 + i];
+  }
+}
+
+template <typename T, int V>
+__global__ void __launch_bounds__(1024)
+postnorm_residual_kernel(float* __restrict__ x, const T* __restrict__ a, const float* __restrict__ wa,
+                         const T* __restrict__ b, const float* __restrict__ wb, float bscale, const T* __restrict__ e,
+                         const float* __restrict__ ecoef, int K, const float* __restrict__ idw,
+                         const float* __restrict__ w, float eps, float mult, const float* __restrict__ wn,
+                         T* __restrict__ out, int H) {
+  __shared__ float red[32];
+  const size_t t = blockIdx.x, row = t * H;
+  const float ic = idw ? idw[t] : 0.f, invH = 1.f / (float)H;
+  float xv[PN_PER][V], y[PN_PER][V];
+  float sa = 0.f, sb = 0.f;
+  float bv[PN_PER][V];
+#pragma unroll
+  for (int u = 0; u < PN_PER; ++u) {
+    const int i = (threadIdx.x + blockDim.x * u) * V;
+#pragma unroll
+    for (int r = 0; r < V; ++r) xv[u][r] = y[u][r] = bv[u][r] = 0.f;
+    if (i >= H) continue;
+    ldv<float, V>(x + row + i, xv[u]);
+    if (w == nullptr) continue;
+    if (a) ldv<T, V>(a + row + i, y[u]);
+    if (b) ldv<T, V>(b + row + i, bv[u]);
+    for (int k = 0; k < K; ++k) {
+      const float c = ecoef[t * K + k];
+      if (c == 0.f) continue;  // (an identity choice: its row of e was never written)
+      float ev[V];
+      ldv<T, V>(e + (t * K + k) * H + i, ev);
+#pragma unroll
+      for (int r = 0; r < V; ++r) y[u][r] = fmaf(c, ev[r], y[u][r]);
+    }
+    if (idw) {
+#pragma unroll
+      for (int r = 0; r < V; ++r) y[u][r] = fmaf(ic, xv[u][r], y[u][r]);
+    }
+#pragma unroll
+    for (int r = 0; r < V; ++r) {
+      sa = fmaf(y[u][r], y[u][r], sa);
+      sb = fmaf(bv[u][r], bv[u][r], sb);
+    }
+  }
+  if (w != nullptr) {
+    block_sum2(sa, sb, red);
+    if (wa != nullptr) {
+      const float ra = bscale / sqrtf(sa * invH + eps), rb = bscale / sqrtf(sb * invH + eps);
+      sa = 0.f;
+      sb = 0.f;
+#pragma unroll
+      for (int u = 0; u < PN_PER; ++u) {
+        const int i = (threadIdx.x + blockDim.x * u) * V;
+        if (i >= H) continue;
+        float va[V], vb[V];
+        ldv<float, V>(wa + i, va);
+        if (b) ldv<float, V>(wb + i, vb);
+#pragma unroll
+        for (int r = 0; r < V; ++r) {
+          y[u][r] = y[u][r] * ra * va[r] + (b ? bv[u][r] * rb * vb[r] : 0.f);
+          sa = fmaf(y[u][r], y[u][r], sa);
+        }
+      }
+      block_sum2(sa, sb, red);
+    }
+    const float ry = mult / sqrtf(sa * invH + eps);
+    sa = 0.f;
+    sb = 0.f;
+#pragma unroll
+    for (int u = 0; u < PN_PER; ++u) {
+      const int i = (threadIdx.x + blockDim.x * u) * V;
+      if (i >= H) continue;
+      float vw[V];
+      ldv<float, V>(w + i, vw);
+#pragma unroll
+      for (int r = 0; r < V; ++r) {
+        xv[u][r] += y[u][r] * ry * vw[r];
+        sa = fmaf(xv[u][r], xv[u][r], sa);
+      }
+      stv<float, V>(x + row + i, xv[u]);
+    }
+  } else if (wn != nullptr) {
+#pragma unroll
+    for (int u = 0; u < PN_PER; ++u)
+#pragma unroll
+      for (int r = 0; r < V; ++r) sa = fmaf(xv[u][r], xv[u][r], sa);
+  }
+  if (out == nullptr) return;
+  float rx = 1.f;
+  if (wn != nullptr) {
+    block_sum2(sa, sb, red);
+    rx = 1.f / sqrtf(sa * invH + eps);
+  }
+#pragma unroll
+  for (int u = 0; u < PN_PER; ++u) {
+    const int i = (threadIdx.x + blockDim.x * u) * V;
+    if (i >= H) continue;
+    if (wn != nullptr) {
+      float vn[V];
+      ldv<float, V>(wn + i, vn);
+#pragma unroll
+      for (int r = 0; r < V; ++r) xv[u][r] *= rx * vn[r];
+    }
+    stv<T, V>(out + row + i, xv[u]);
+  }
+}
+
 }  // namespace grag
 
 using namespace grag;
@@ -737,8 +912,11 @@ GRAG_API int grag_moe_max_rows() { return RT_MAXR; }
 GRAG_API int grag_moe_max_top() { return RT_MAXTOP; }
 
 GRAG_API hipError_t grag_moe_route(const void* h, int ld, const float* wr, int W, int E, int R, int top, int ngroups,
-                                   int keep, int* ids, float* wts, float* sgate, int T_, int dt, hipStream_t st) {
+                                   int keep, int* ids, float* wts, float* sgate, int T_, int dt, const float* corr,
+                                   int nid, float* idw, hipStream_t st) {
+  const RouteExtra rx{corr, nid, idw};
   if (T_ <= 0) return hipSuccess;
+  if (nid < 0 || nid > E || (nid > 0 && idw == nullptr)) return hipErrorInvalidValue;
   if (E < 1 || R < E || R > RT_MAXR || top < 1 || top > RT_MAXTOP || top > E || ngroups < 1 || E % ngroups ||
       keep < 1 || keep > ngroups)
     return hipErrorInvalidValue;
@@ -747,7 +925,7 @@ GRAG_API hipError_t grag_moe_route(const void* h, int ld, const float* wr, int W
                   (reinterpret_cast<uintptr_t>(wr) & 15) == 0;
   if (T_ <= 128) {  // decode rows, short portions
     DT_DISPATCH(dt, hipLaunchKernelGGL(moe_route_rows_kernel<T>, dim3(T_), dim3(256), 0, st, (const T*)h, ld, wr, W, E, R,
-                                       top, ngroups, keep, ids, wts, sgate, vec);)
+                                       top, ngroups, keep, ids, wts, sgate, vec, rx);)
     return hipGetLastError();
   }
   DT_DISPATCH(dt, {
@@ -757,7 +935,7 @@ GRAG_API hipError_t grag_moe_route(const void* h, int ld, const float* wr, int W
       if (e != hipSuccess) return e;
     }
     hipLaunchKernelGGL(moe_route_kernel<T>, dim3((T_ + RT_TOK - 1) / RT_TOK), dim3(256), bytes, st, (const T*)h, ld, wr,
-                       W, E, R, top, ngroups, keep, ids, wts, sgate, T_, vec);
+                       W, E, R, top, ngroups, keep, ids, wts, sgate, T_, vec, rx);
   })
   return hipGetLastError();
 }
@@ -779,14 +957,14 @@ GRAG_API hipError_t grag_moe_table_route(const int* tok, const int* table, int n
 }
 
 // rows = T * top sorted rows.  gated 1: a = h [T][lda], w = [E][2N][K], out [rows][N]; gated 0: a = [rows][lda] sorted,
-// w = [E][N][K], out [rows][ldo] in (token, choice) order; gated 2: one matrix per head (E heads, top = tokens, rows =
+// w = [E][N][K], out [rows][ldo] in (token, choice) order; gated 3: as 1 with one branch, w = [E][N][K]; gated 2: one matrix per head (E heads, top = tokens, rows =
 // tokens * E): a = [tokens * E][lda], w = [E][N][K], out [tokens * E][ldo], offs / order unused.
 GRAG_API hipError_t grag_moe_gemm(const void* a, int lda, const void* w, const int* offs, const int* order, int rows,
                                   int E, int top, int N, int K, void* out, int ldo, int gated, int dt, float limit,
                                   float alpha, float shift, const void* gate, int gate_ld, hipStream_t st) {
   if (rows <= 0) return hipSuccess;
   const int tiles = (rows + MG_M - 1) / MG_M + E;  // every expert may end on a partial tile
-  if (tiles > 65535 || E < 1 || top < 1 || gated < 0 || gated > 2) return hipErrorInvalidValue;
+  if (tiles > 65535 || E < 1 || top < 1 || gated < 0 || gated > 3) return hipErrorInvalidValue;
   if (gated == 2 ? rows != E * top : (offs == nullptr || order == nullptr)) return hipErrorInvalidValue;
   const MoeEpi ep{limit, alpha, shift, gate, gate_ld};
   const dim3 grid((N + MG_N - 1) / MG_N, tiles);
@@ -797,6 +975,8 @@ GRAG_API hipError_t grag_moe_gemm(const void* a, int lda, const void* w, const i
       hipLaunchKernelGGL((KERN<1>), GRID, dim3(256), 0, st, A, lda, W, offs, order, E, top, N, K, O, ldo, ep);       \
     else if (gated == 2)                                                                                             \
       hipLaunchKernelGGL((KERN<2>), GRID, dim3(256), 0, st, A, lda, W, offs, order, E, top, N, K, O, ldo, ep);       \
+    else if (gated == 3)                                                                                             \
+      hipLaunchKernelGGL((KERN<3>), GRID, dim3(256), 0, st, A, lda, W, offs, order, E, top, N, K, O, ldo, ep);       \
     else                                                                                                             \
       hipLaunchKernelGGL((KERN<0>), GRID, dim3(256), 0, st, A, lda, W, offs, order, E, top, N, K, O, ldo, ep);       \
   }
@@ -818,6 +998,9 @@ GRAG_API hipError_t grag_moe_gemm(const void* a, int lda, const void* w, const i
                          top, N, K, (T*)out, ldo, ep);
     else if (gated == 2)
       hipLaunchKernelGGL((moe_gemm_kernel<T, 2>), grid, dim3(256), 0, st, (const T*)a, lda, (const T*)w, offs, order, E,
+                         top, N, K, (T*)out, ldo, ep);
+    else if (gated == 3)
+      hipLaunchKernelGGL((moe_gemm_kernel<T, 3>), grid, dim3(256), 0, st, (const T*)a, lda, (const T*)w, offs, order, E,
                          top, N, K, (T*)out, ldo, ep);
     else
       hipLaunchKernelGGL((moe_gemm_kernel<T, 0>), grid, dim3(256), 0, st, (const T*)a, lda, (const T*)w, offs, order, E,
@@ -845,5 +1028,33 @@ GRAG_API hipError_t grag_residual_rmsnorm(float* x, float keep, const void* a, c
   DT_DISPATCH(dt, hipLaunchKernelGGL(residual_rmsnorm_kernel<T>, dim3(T_), dim3(256), 0, st, x, keep, (const T*)a,
                                      (const T*)b, bcoef, (const T*)e, ecoef, e ? K : 0, w, eps, (T*)out, (T*)raw,
                                      raw_ld, H, (const T*)gate, gate_ld, gbias, mult);)
+  return hipGetLastError();
+}
+
+GRAG_API int grag_postnorm_max_width() { return 1024 * PN_PER; }
+
+GRAG_API hipError_t grag_postnorm_residual(float* x, const void* a, const float* wa, const void* b, const float* wb,
+                                           float bscale, const void* e, const float* ecoef, int K, const float* idw,
+                                           const float* w, float eps, float mult, const float* wn, void* out, int T_,
+                                           int H, int dt, hipStream_t st) {
+  if (T_ <= 0) return hipSuccess;
+  if (H < 1 || K < 0 || (K > 0 && (e == nullptr || ecoef == nullptr)) || (b != nullptr && (wa == nullptr || wb == nullptr)) ||
+      (wa != nullptr && (a == nullptr || K > 0 || idw != nullptr)))
+    return hipErrorInvalidValue;
+  auto al16 = [](const void* p) { return (reinterpret_cast<uintptr_t>(p) & 15) == 0; };
+  const bool vec = H % 4 == 0 && al16(x) && al16(a) && al16(wa) && al16(b) && al16(wb) && al16(e) && al16(w) && al16(wn) &&
+                   al16(out);
+  const int groups = vec ? H / 4 : H;
+  if (groups > 1024 * PN_PER) return hipErrorInvalidValue;
+  // two groups per thread where that fills whole waves, up to 1024 threads
+  const int threads = min(1024, max(64, (((groups + 1) / 2 + 63) / 64) * 64));
+  DT_DISPATCH(dt, {
+    if (vec)
+      hipLaunchKernelGGL((postnorm_residual_kernel<T, 4>), dim3(T_), dim3(threads), 0, st, x, (const T*)a, wa, (const T*)b,
+                         wb, bscale, (const T*)e, ecoef, K, idw, w, eps, mult, wn, (T*)out, H);
+    else
+      hipLaunchKernelGGL((postnorm_residual_kernel<T, 1>), dim3(T_), dim3(threads), 0, st, x, (const T*)a, wa, (const T*)b,
+                         wb, bscale, (const T*)e, ecoef, K, idw, w, eps, mult, wn, (T*)out, H);
+  })
   return hipGetLastError();
 }

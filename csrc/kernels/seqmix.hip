@@ -105,14 +105,16 @@ __global__ void dyt_residual_vec_kernel(const T* __restrict__ y, float a1, const
 // q_out [T, H*d] = rotated q; k_cache [nblk, G, BS, d] <- rotated k; v_cache [nblk, G, BS, vd] <- v / rms(v).
 // Rotation: the first rd dims of a head, dim i paired with i + rd/2 (flags bit 0 set: dim 2i paired with 2i + 1, the
 // interleaved layout); table row p = cos[0:rd/2] | sin[0:rd/2] (fp32).  flags bit 1 set: the values are stored as
-// they are (no RMS division).
+// they are (no RMS division).  bias (null: none) [ld] fp32 is added to the projection first, by column; with qw / kw
+// [d] fp32 every q / k head is then divided by its RMS and multiplied by them, before the rotation.
 // grid (T, ceil((H + G + G) / 4)), 256 threads: one wave per (token, head): q heads, then k heads, then v heads.
 template <typename T>
 __global__ void rope_vnorm_store_kernel(const T* __restrict__ proj, int ld, int qoff, int koff, int voff,
                                         const int* __restrict__ positions, const float* __restrict__ table,
                                         int table_rows, const int* __restrict__ slot_mapping, T* __restrict__ q_out,
                                         T* __restrict__ k_cache, T* __restrict__ v_cache, int H, int G, int d, int vd,
-                                        int rd, int BS, long nslots, float eps, int flags) {
+                                        int rd, int BS, long nslots, float eps, int flags, const float* __restrict__ bias,
+                                        const float* __restrict__ qw, const float* __restrict__ kw) {
   const int t = blockIdx.x, hb = blockIdx.y * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
   if (hb >= H + 2 * G) return;
   const T* row = proj + (size_t)t * ld;
@@ -122,15 +124,19 @@ __global__ void rope_vnorm_store_kernel(const T* __restrict__ proj, int ld, int 
   if (hb >= H + G) {  // a value head: RMS over vd in fp32
     const int g = hb - H - G;
     const T* x = row + voff + g * vd;
-    float ss = 0.f;
-    for (int i = lane; i < vd; i += 64) {
-      const float v = ldf(x + i);
-      ss += v * v;
+    const float* xb = bias ? bias + voff + g * vd : nullptr;
+    float r = 1.f;
+    if (!(flags & 2)) {
+      float ss = 0.f;
+      for (int i = lane; i < vd; i += 64) {
+        const float v = ldf(x + i) + (xb ? xb[i] : 0.f);
+        ss += v * v;
+      }
+      r = 1.f / sqrtf(wave_sum(ss) / (float)vd + eps);
     }
-    ss = wave_sum(ss);
-    const float r = (flags & 2) ? 1.f : 1.f / sqrtf(ss / (float)vd + eps);
     if (store)
-      for (int i = lane; i < vd; i += 64) stf(v_cache + (((size_t)blk * G + g) * BS + off) * vd + i, ldf(x + i) * r);
+      for (int i = lane; i < vd; i += 64)
+        stf(v_cache + (((size_t)blk * G + g) * BS + off) * vd + i, (ldf(x + i) + (xb ? xb[i] : 0.f)) * r);
     return;
   }
   const int pos = positions[t];
@@ -142,17 +148,32 @@ __global__ void rope_vnorm_store_kernel(const T* __restrict__ proj, int ld, int 
   const T* x = row + (isq ? qoff : koff) + hh * d;
   if (!isq && !store) return;
   T* dst = isq ? q_out + ((size_t)t * H + hh) * d : k_cache + (((size_t)blk * G + hh) * BS + off) * d;
+  const float* xb = bias ? bias + (isq ? qoff : koff) + hh * d : nullptr;
+  const float* nw = isq ? qw : kw;
+  float r = 1.f;
+  if (nw) {
+    float ss = 0.f;
+    for (int i = lane; i < d; i += 64) {
+      const float v = ldf(x + i) + (xb ? xb[i] : 0.f);
+      ss += v * v;
+    }
+    r = 1.f / sqrtf(wave_sum(ss) / (float)d + eps);
+  }
+  auto at = [&](int i) {
+    const float v = ldf(x + i) + (xb ? xb[i] : 0.f);
+    return nw ? v * r * nw[i] : v;
+  };
   for (int i = lane; i < d; i += 64) {
-    float v = ldf(x + i);
+    float v = at(i);
     if (i < rd && pos_ok && (flags & 1)) {  // adjacent pairs: (2j, 2j + 1) turned by angle j
       const int j = i >> 1;
-      v = (i & 1) ? v * cs[j] + ldf(x + i - 1) * cs[half + j] : v * cs[j] - ldf(x + i + 1) * cs[half + j];
+      v = (i & 1) ? v * cs[j] + at(i - 1) * cs[half + j] : v * cs[j] - at(i + 1) * cs[half + j];
     } else if (i < rd && pos_ok) {
       if (i < half) {
-        v = v * cs[i] - ldf(x + i + half) * cs[half + i];
+        v = v * cs[i] - at(i + half) * cs[half + i];
       } else {
         const int j = i - half;
-        v = v * cs[j] + ldf(x + j) * cs[half + j];
+        v = v * cs[j] + at(j) * cs[half + j];
       }
     }
     stf(dst + i, v);
@@ -166,8 +187,9 @@ __global__ void rope_vnorm_store_kernel(const T* __restrict__ proj, int ld, int 
 // head); `chunk` > 0 confines a query at position i to the keys j of its own aligned block of `chunk` positions,
 // floor(j / chunk) == floor(i / chunk) (and j <= i); `hgate` [T][gate_ld] holds one logit per (token, head) and the
 // head's output is multiplied by its sigmoid as it is stored; `window` > 0 is sliding-window attention, a query at
-// position i sees key j only when 0 <= i - j < window; `softcap` > 0 sends every scaled score s through
-// softcap * tanh(s / softcap) before the softmax.
+// position i sees key j only when 0 <= i - j < window; `keep` > 0: the keys j < keep stay visible to every query behind
+// them, whatever the window or block hides; `softcap` > 0 sends every scaled score s through softcap * tanh(s / softcap)
+// before the softmax.
 struct AttnExtra {
   const float* hscale;
   const void* hgate;
@@ -175,15 +197,26 @@ struct AttnExtra {
   int chunk;
   int window;
   float softcap;
+  int keep;
 };
 template <typename T>
 __device__ __forceinline__ float head_gate(const AttnExtra& ex, size_t row, int h) {
   return ex.hgate ? sigmoid_acc(ldf(reinterpret_cast<const T*>(ex.hgate) + row * ex.gate_ld + h)) : 1.f;
 }
-// the first key the query at position `pos` sees (never falls as pos grows)
+// the first key of the window / block of the query at position `pos` (never falls as pos grows)
 __device__ __forceinline__ int chunk_start(const AttnExtra& ex, int pos) {
   const int lo = ex.chunk > 0 ? pos - pos % ex.chunk : 0;
   return ex.window > 0 ? max(lo, pos - ex.window + 1) : lo;
+}
+// Key tiles of a query tile whose first window starts at `lo`: with kept keys the walk starts at key 0 and leaps from the
+// end of the last tile that holds a kept key to `lo` (a tile never overlaps the one before it, and the masks hide what
+// lies between).
+__device__ __forceinline__ int first_tile(const AttnExtra& ex, int beg, int lo) {
+  return beg < ex.keep ? beg : max(beg, lo);
+}
+__device__ __forceinline__ int next_tile(const AttnExtra& ex, int k0, int kt, int lo) {
+  const int n = k0 + kt;
+  return n >= ex.keep && n < lo ? lo : n;
 }
 __device__ __forceinline__ float cap_score(const AttnExtra& ex, float s) {
   return ex.softcap > 0.f ? ex.softcap * tanhf(s / ex.softcap) : s;
@@ -232,7 +265,8 @@ sink_attn_prefill_kernel(const T* __restrict__ q, const T* __restrict__ k_cache,
   const int last_q = min(q0 + QT, qlen) - 1;
   const int nkeys = min(ctx, pos0 + last_q + 1);
   const int* bt = block_tables + (size_t)seq * bt_stride;
-  for (int k0 = chunk_start(ex, pos0 + q0); k0 < nkeys; k0 += KT) {  // (the tile's first query has the earliest block)
+  const int klo = chunk_start(ex, pos0 + q0);  // (the tile's first query has the earliest window)
+  for (int k0 = first_tile(ex, 0, klo); k0 < nkeys; k0 = next_tile(ex, k0, KT, klo)) {
     __syncthreads();
     const int kn = min(KT, nkeys - k0);
     for (int idx = threadIdx.x; idx < kn * d; idx += 256) {
@@ -270,7 +304,8 @@ sink_attn_prefill_kernel(const T* __restrict__ q, const T* __restrict__ k_cache,
 #pragma unroll
     for (int n = 0; n < SA_NQ; ++n) {
       const int tq = q0 + wid * SA_NQ + n;
-      const bool vis = lane < kn && tq < qlen && (k0 + lane) <= pos0 + tq && (k0 + lane) >= chunk_start(ex, pos0 + tq);
+      const bool vis = lane < kn && tq < qlen && (k0 + lane) <= pos0 + tq &&
+                       ((k0 + lane) >= chunk_start(ex, pos0 + tq) || k0 + lane < ex.keep);
       const float sc = vis ? cap_score(ex, s[n] * scale) : -INFINITY;
       const float mn = fmaxf(m[n], wave_max(sc));
       const float p = vis ? expf(sc - mn) : 0.f;
@@ -366,7 +401,8 @@ sink_attn_prefill_mfma_kernel(const bf16* __restrict__ q, const bf16* __restrict
   const int wave_qmax = pos0 + min(q0 + wid * 16 + 15, qlen - 1);
   // aligned blocks of ex.chunk positions: the tile loop starts at the block of the workgroup's first query; a wave skips
   // the tiles before the block of ITS first query, and masks against each query's own block start
-  const int kfirst = chunk_start(ex, pos0 + q0);
+  const int klo = chunk_start(ex, pos0 + q0);
+  const int kfirst = first_tile(ex, 0, klo);
   const int wave_cmin = chunk_start(ex, pos0 + q0 + wid * 16), wave_cmax = chunk_start(ex, wave_qmax);
   const int cstart = chunk_start(ex, q_ok ? qpos : pos0 + q0);
   const int* bt = block_tables + (size_t)seq * bt_stride;
@@ -378,18 +414,22 @@ sink_attn_prefill_mfma_kernel(const bf16* __restrict__ q, const bf16* __restrict
     tile_load(kreg, k_cache, blk, rc.off, d, G, g, BS);
     tile_load(vreg, v_cache, blk, rc.off, vd, G, g, BS, v_ld);
   }
-  for (int k0 = kfirst; k0 < nkeys; k0 += KT) {
+  int knext;
+  for (int k0 = kfirst; k0 < nkeys; k0 = knext) {
+    knext = next_tile(ex, k0, KT, klo);
     __syncthreads();
     tile_store(kreg, Ks, d, kstride);
     tile_store_v4(vreg, Vs, vd, vstride);
     __syncthreads();
-    if (k0 + KT < nkeys) {  // the next tile's loads fly while this one is computed
-      rc.advance(BS);
-      const int blk = tile_block(rc, bt, k0 + KT + (threadIdx.x >> 2), nkeys, nblocks, ERR_BLOCK_PREFILL);
+    if (knext < nkeys) {  // the next tile's loads fly while this one is computed
+      if (knext == k0 + KT) rc.advance(BS);
+      else rc.init(knext + (threadIdx.x >> 2), BS);
+      const int blk = tile_block(rc, bt, knext + (threadIdx.x >> 2), nkeys, nblocks, ERR_BLOCK_PREFILL);
       tile_load(kreg, k_cache, blk, rc.off, d, G, g, BS);
       tile_load(vreg, v_cache, blk, rc.off, vd, G, g, BS, v_ld);
     }
-    if (k0 > wave_qmax || k0 + KT <= wave_cmin) continue;  // every key lies after, or in a block before, this wave's queries
+    // every key lies after, or in a block / before the window of, this wave's queries (and none is kept)
+    if (k0 > wave_qmax || (k0 + KT <= wave_cmin && k0 >= ex.keep)) continue;
     f32x4_t st[4];
 #pragma unroll
     for (int n = 0; n < 4; ++n) {
@@ -410,7 +450,7 @@ sink_attn_prefill_mfma_kernel(const bf16* __restrict__ q, const bf16* __restrict
     float tmax = -INFINITY;
     // a tile wholly at or before the wave's first query (and inside the context) needs no mask
     const bool interior = k0 + KT - 1 <= pos0 + q0 + wid * 16 && k0 + KT <= nkeys && q0 + wid * 16 + 15 < qlen &&
-                          k0 >= wave_cmax;
+                          (k0 >= wave_cmax || k0 + KT <= ex.keep);
     if (ex.softcap > 0.f) {  // cap in the natural domain, then to log2
       const float s1 = scale * (ex.hscale ? ex.hscale[h] : 1.f), ic = 1.f / ex.softcap, c2 = ex.softcap * LOG2E;
 #pragma unroll
@@ -432,7 +472,7 @@ sink_attn_prefill_mfma_kernel(const bf16* __restrict__ q, const bf16* __restrict
 #pragma unroll
         for (int i = 0; i < 4; ++i) {
           const int key = k0 + 16 * n + 4 * quad + i;
-          const bool vis = q_ok && key < nkeys && key <= qpos && key >= cstart;
+          const bool vis = q_ok && key < nkeys && key <= qpos && (key >= cstart || key < ex.keep);
           st[n][i] = vis ? st[n][i] * sc2 : -INFINITY;
           tmax = fmaxf(tmax, st[n][i]);
         }
@@ -552,7 +592,8 @@ sink_attn_decode_mfma_kernel(const bf16* __restrict__ q, const bf16* __restrict_
 #pragma unroll
   for (int v = 0; v < NVM; ++v) acc[v] = f32x4_t{0.f, 0.f, 0.f, 0.f};
   const int kend = SIG ? ctx : nsplit > 1 ? min(ctx, sp * split_len + split_len) : ctx;
-  const int kbeg = SIG ? max(0, ctx - window) : max(nsplit > 1 ? sp * split_len : 0, chunk_start(ex, ctx - 1));
+  const int klo = SIG ? max(0, ctx - window) : chunk_start(ex, ctx - 1);
+  const int kbeg = SIG ? klo : first_tile(ex, nsplit > 1 ? sp * split_len : 0, klo);
   const int* bt = block_tables + (size_t)seq * bt_stride;
   bf16x8_t kreg[NKM / 2], vreg[NVM / 2];
   RowCursor rc;
@@ -562,14 +603,17 @@ sink_attn_decode_mfma_kernel(const bf16* __restrict__ q, const bf16* __restrict_
     tile_load(kreg, k_cache, blk, rc.off, d, G, g, BS);
     tile_load(vreg, v_cache, blk, rc.off, vd, G, g, BS, v_ld);
   }
-  for (int k0 = kbeg; k0 < kend; k0 += KT) {
+  int knext;
+  for (int k0 = kbeg; k0 < kend; k0 = knext) {
+    knext = SIG ? k0 + KT : next_tile(ex, k0, KT, klo);
     __syncthreads();
     tile_store(kreg, Ks, d, kstride);
     tile_store_v4(vreg, Vs, vd, vstride);
     __syncthreads();
-    if (k0 + KT < kend) {
-      rc.advance(BS);
-      const int blk = tile_block(rc, bt, k0 + KT + (threadIdx.x >> 2), kend, nblocks, ERR_BLOCK_DECODE);
+    if (knext < kend) {
+      if (knext == k0 + KT) rc.advance(BS);
+      else rc.init(knext + (threadIdx.x >> 2), BS);
+      const int blk = tile_block(rc, bt, knext + (threadIdx.x >> 2), kend, nblocks, ERR_BLOCK_DECODE);
       tile_load(kreg, k_cache, blk, rc.off, d, G, g, BS);
       tile_load(vreg, v_cache, blk, rc.off, vd, G, g, BS, v_ld);
     }
@@ -599,7 +643,8 @@ sink_attn_decode_mfma_kernel(const bf16* __restrict__ q, const bf16* __restrict_
       float tmax = -INFINITY;
 #pragma unroll
       for (int i = 0; i < 4; ++i) {
-        const bool vis = col_ok && 16 * wid + 4 * quad + i < kn;
+        const int kk = 16 * wid + 4 * quad + i;
+        const bool vis = col_ok && kk < kn && (k0 + kk >= klo || k0 + kk < ex.keep);
         st[i] = vis ? cap_score(ex, st[i] * scale) : -INFINITY;
         tmax = fmaxf(tmax, st[i]);
       }
@@ -748,9 +793,12 @@ sink_attn_decode_vec_kernel(const bf16* __restrict__ q, const bf16* __restrict__
   float* pw = Ps + wid * 64;
   const int ntiles = (ctx + 63) >> 6;
   const int d8 = d >> 3;
-  for (int t = (kbeg >> 6) + wid; t < ntiles; t += 4) {
+  const int kept = min((ex.keep + 63) >> 6, ntiles);  // tiles that hold kept keys, then those of the window
+  const int wtile = max(kbeg >> 6, kept);
+  for (int n = wid; n < kept + ntiles - wtile; n += 4) {
+    const int t = n < kept ? n : wtile + n - kept;
     const int key = t * 64 + lane;
-    const bool vis = key < ctx && key >= kbeg;
+    const bool vis = key < ctx && (key >= kbeg || key < ex.keep);
     float s = 0.f;
     if (vis) {
       int blk = bt[key / BS];
@@ -778,7 +826,7 @@ sink_attn_decode_vec_kernel(const bf16* __restrict__ q, const bf16* __restrict__
       const int j = 2 * lane + 128 * c;
       float a0 = acc[c][0] * alpha, a1 = acc[c][1] * alpha;
       if (j < vd) {
-        for (int kk = max(0, kbeg - t * 64); kk < kn; ++kk) {
+        for (int kk = n < kept ? 0 : max(0, kbeg - t * 64); kk < kn; ++kk) {
           const int key2 = t * 64 + kk;
           int b2 = bt[key2 / BS];
           if (b2 < 0 || b2 >= nblocks) b2 = 0;
@@ -850,9 +898,12 @@ sink_attn_decode_kernel(const T* __restrict__ q, const T* __restrict__ k_cache, 
   const int* bt = block_tables + (size_t)seq * bt_stride;
   float* pw = Ps + wid * 64;
   const int ntiles = (ctx + 63) >> 6;
-  for (int t = (kbeg >> 6) + wid; t < ntiles; t += 4) {
+  const int kept = min((ex.keep + 63) >> 6, ntiles);  // tiles that hold kept keys, then those of the window
+  const int wtile = max(kbeg >> 6, kept);
+  for (int n = wid; n < kept + ntiles - wtile; n += 4) {
+    const int t = n < kept ? n : wtile + n - kept;
     const int key = t * 64 + lane;
-    const bool vis = key < ctx && key >= kbeg;
+    const bool vis = key < ctx && (key >= kbeg || key < ex.keep);
     float s = 0.f;
     int blk = 0;
     if (vis) {
@@ -877,7 +928,7 @@ sink_attn_decode_kernel(const T* __restrict__ q, const T* __restrict__ k_cache, 
       const int j = lane + 64 * c;
       float a = acc[c] * alpha;
       if (j < vd) {
-        for (int kk = max(0, kbeg - t * 64); kk < kn; ++kk) {
+        for (int kk = n < kept ? 0 : max(0, kbeg - t * 64); kk < kn; ++kk) {
           const int key2 = t * 64 + kk;
           int b2 = bt[key2 / BS];
           if (b2 < 0 || b2 >= nblocks) b2 = 0;
@@ -1241,6 +1292,27 @@ __global__ void clamped_glu_vec_kernel(const bf16* __restrict__ gu, bf16* __rest
   *reinterpret_cast<bf16x8_t*>(out + t * F + i) = o;
 }
 
+// ------------------------------------------------------------------------------------------------ squared relu
+// x [n], in place: max(x, 0)^2.  bf16 with n % 8 == 0 and a 16-byte aligned start: 8 elements per thread.
+template <typename T>
+__global__ void relu2_kernel(T* __restrict__ x, size_t n) {
+  const size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
+  if (i >= n) return;
+  const float v = fmaxf(ldf(x + i), 0.f);
+  stf(x + i, v * v);
+}
+__global__ void relu2_vec_kernel(bf16* __restrict__ x, size_t n) {
+  const size_t i = ((size_t)blockIdx.x * blockDim.x + threadIdx.x) * 8;
+  if (i >= n) return;
+  bf16x8_t v8 = *reinterpret_cast<const bf16x8_t*>(x + i);
+#pragma unroll
+  for (int e = 0; e < 8; ++e) {
+    const float v = fmaxf(bits2f(v8[e]), 0.f);
+    v8[e] = f2bits(v * v);
+  }
+  *reinterpret_cast<bf16x8_t*>(x + i) = v8;
+}
+
 }  // namespace grag
 
 using namespace grag;
@@ -1280,12 +1352,13 @@ GRAG_API hipError_t grag_dyt_residual(const void* y, float a1, const float* w1, 
 GRAG_API hipError_t grag_rope_vnorm_store(const void* proj, int ld, int qoff, int koff, int voff, const int* positions,
                                           const float* table, int table_rows, const int* slot_mapping, void* q_out,
                                           void* k_cache, void* v_cache, int T_, int H, int G, int d, int vd, int rd,
-                                          int BS, long nslots, float eps, int dt, int flags, hipStream_t st) {
+                                          int BS, long nslots, float eps, int dt, int flags, const float* bias,
+                                          const float* qw, const float* kw, hipStream_t st) {
   if (T_ <= 0) return hipSuccess;
   if (H + 2 * G > 4 * 65535) return hipErrorInvalidValue;
   DT_DISPATCH(dt, hipLaunchKernelGGL(rope_vnorm_store_kernel<T>, dim3(T_, (H + 2 * G + 3) / 4), dim3(256), 0, st, (const T*)proj, ld, qoff,
                                      koff, voff, positions, table, table_rows, slot_mapping, (T*)q_out, (T*)k_cache,
-                                     (T*)v_cache, H, G, d, vd, rd, BS, nslots, eps, flags);)
+                                     (T*)v_cache, H, G, d, vd, rd, BS, nslots, eps, flags, bias, qw, kw);)
   return hipGetLastError();
 }
 
@@ -1306,8 +1379,8 @@ GRAG_API hipError_t grag_sink_attn_prefill(const void* q, const void* k_cache, c
                                            const int* ctx_len, const float* sinks, int nseq, int max_q_len, int H,
                                            int G, int d, int vd, int BS, float scale, float out_scale, int nblocks,
                                            int dt, int v_ld, const float* hscale, const void* hgate, int gate_ld,
-                                           int chunk, int window, float softcap, hipStream_t st) {
-  const AttnExtra ex{hscale, hgate, gate_ld, chunk, window, softcap};
+                                           int chunk, int window, float softcap, int keep, hipStream_t st) {
+  const AttnExtra ex{hscale, hgate, gate_ld, chunk, window, softcap, chunk > 0 || window > 0 ? keep : 0};
   // v_ld: elements from one cached value row to the next (vd, or more when the value rows are the head of wider rows)
   if (nseq <= 0 || max_q_len <= 0) return hipSuccess;
   if (vd > 64 * SA_VC || G <= 0 || H % G || v_ld < vd) return hipErrorInvalidValue;
@@ -1360,8 +1433,8 @@ GRAG_API hipError_t grag_sink_attn_decode(const void* q, const void* k_cache, co
                                           float scale, float out_scale, int nblocks, int dt, int nsplit,
                                           int split_len, float* part_o, float* part_ml, int v_ld, const float* hscale,
                                           const void* hgate, int gate_ld, int chunk, int window, float softcap,
-                                          hipStream_t st) {
-  const AttnExtra ex{hscale, hgate, gate_ld, chunk, window, softcap};
+                                          int keep, hipStream_t st) {
+  const AttnExtra ex{hscale, hgate, gate_ld, chunk, window, softcap, chunk > 0 || window > 0 ? keep : 0};
   if (nseq <= 0) return hipSuccess;
   if (vd > 64 * SA_VC || G <= 0 || H % G || v_ld < vd) return hipErrorInvalidValue;
   if (dt == 0 && v_ld % 8 == 0 && (reinterpret_cast<uintptr_t>(v_cache) & 15) == 0 && d % 16 == 0 && vd % 16 == 0 && d <= 256 && vd <= 256 && G * ((H / G + 15) / 16) <= 65535 &&
@@ -1434,7 +1507,7 @@ GRAG_API hipError_t grag_window_decode_mfma(const void* q, const void* k_cache, 
     hipLaunchKernelGGL((sink_attn_decode_mfma_kernel<NK, NV, 1>), mgrid, dim3(256), mb, st, (const bf16*)q,          \
                        (const bf16*)k_cache, (const bf16*)v_cache, (bf16*)out, out_ld, block_tables, bt_stride,      \
                        ctx_len, bias, H, G, d, vd, BS, scale, 1.f, nblocks, 1, 0, (float*)nullptr, (float*)nullptr,  \
-                       window, (const bf16*)gate, gate_ld, vd, AttnExtra{nullptr, nullptr, 0, 0, 0, 0.f});                   \
+                       window, (const bf16*)gate, gate_ld, vd, AttnExtra{nullptr, nullptr, 0, 0, 0, 0.f, 0});                 \
   }
   if (d <= 64 && vd <= 64) SW_MFMA(4, 4)
   else SW_MFMA(8, 8)
@@ -1555,5 +1628,15 @@ GRAG_API hipError_t grag_clamped_glu(const void* gu, void* out, int T_, int F, f
   const dim3 grid(T_, (F + 255) / 256);
   DT_DISPATCH(dt, hipLaunchKernelGGL(clamped_glu_kernel<T>, grid, dim3(256), 0, st, (const T*)gu, (T*)out, F, limit,
                                      alpha, shift);)
+  return hipGetLastError();
+}
+
+GRAG_API hipError_t grag_relu2(void* x, int64_t n, int dt, hipStream_t st) {
+  if (n <= 0) return hipSuccess;
+  if (dt == 0 && n % 8 == 0 && (reinterpret_cast<uintptr_t>(x) & 15) == 0) {
+    hipLaunchKernelGGL(relu2_vec_kernel, dim3((unsigned)((n / 8 + 255) / 256)), dim3(256), 0, st, (bf16*)x, (size_t)n);
+    return hipGetLastError();
+  }
+  DT_DISPATCH(dt, hipLaunchKernelGGL(relu2_kernel<T>, dim3((unsigned)((n + 255) / 256)), dim3(256), 0, st, (T*)x, (size_t)n);)
   return hipGetLastError();
 }

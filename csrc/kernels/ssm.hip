@@ -4,6 +4,9 @@
 //   * the scan: per head a state S [N, P] fp32 with a scalar, input-dependent decay per step,
 //       dt_t = softplus(raw_t + bias_h),  S_t = exp(-exp(A_log_h) dt_t) S_(t-1) + dt_t B_t x_t^T,  y_t = S_t^T C_t + D_h x_t
 //     (B, C shared by the heads of a group).  Everything between the convolution's output and y is fp32.
+//   * the scan with a decay per channel AND state number: per channel c a state of N numbers,
+//       dt_t = softplus(W_dt low_t + bias_c),  S_n = exp(dt_t A_(c,n)) S_n + dt_t x_t B_(t,n),  y_t = sum_n S_n C_(t,n) + D_c x_t
+//     (low, B, C: one small projection per token, shared by the channels), the output gated by SiLU(z) as it is stored.
 // Activations are bf16 or fp32 (dt: 0 = bf16, 1 = fp32).  A sequence whose first token of the step sits at position 0
 // starts from zeros instead of its slot's contents, so a slot that is used again needs no reset.
 #include "common.h"
@@ -243,6 +246,224 @@ __global__ void ssm_chunk_prefix_kernel(float* __restrict__ state, const int* __
   Sg[e] = S;
 }
 
+// ------------------------------------------------------------------------------------------------ per-channel scan
+// xc [T][inner]: the convolution's output; low [T][low_ld]: step-size numbers (R) | B (N) | C (N); wdt [inner][Rp], the step
+// sizes' matrix, its rows padded with zeros to Rp (a multiple of 32); A [inner][N] fp32 (negative); z = columns zoff ..
+// of proj [T][ld].  state [slots][inner][N] fp32; out [T][inner] = y * SiLU(z).  grid (ceil(inner / 64), nseq, chunks),
+// 256 threads: thread (channel tid / 4, lane part tid % 4) keeps the state numbers 4 (part + 4 j) .. + 3, j < NPT / 4, in
+// registers (4 NPT >= N; numbers past N have B = C = 0).  Tokens are walked SC_TB at a time:
+//   staging   wave w forms the step sizes of its 16 channels for the 16 tokens -- for bf16 one 16 x 16 matrix-core tile
+//             (operand lane: row lane % 16, k = 8 (lane / 16) .. + 7; result lane: tokens 4 (lane / 16) + i, channel
+//             lane % 16) -- and leaves (dt log2 e, dt x) per (token, channel) in LDS, beside the tokens' B and C rows;
+//   walk      every thread updates its numbers; the four parts of a channel add up their share of y;
+//   store     the lane that formed dt adds D x, gates and stores.
+// Long portions are cut into chunks of `chunk` tokens (a multiple of SC_TB) that run side by side:
+//   MODE 0  the whole portion, from and to the slot's state;
+//   MODE 1  grid.z = chunk: the chunk's own contribution from a zero state -> ws [nseq * maxchunks][inner][N], and the sum
+//           of its step sizes (times log2 e) -> wa [nseq * maxchunks][inner];
+//   (chan_chunk_prefix_kernel turns ws[c] into the state at the START of chunk c and stores the final state;)
+//   MODE 2  grid.z = chunk: the outputs of the chunk's tokens, from the chunk-start state in ws.
+constexpr int SC_TB = 16, SC_CH = 64;
+
+// sum over the 4 lanes of a channel, in every lane
+__device__ __forceinline__ float quad_sum(float v) {
+  v += __int_as_float(__builtin_amdgcn_mov_dpp(__float_as_int(v), 0xB1, 0xf, 0xf, true));  // lanes 1 0 3 2
+  v += __int_as_float(__builtin_amdgcn_mov_dpp(__float_as_int(v), 0x4E, 0xf, 0xf, true));  // lanes 2 3 0 1
+  return v;
+}
+
+template <typename T, int NPT, int MODE>
+__global__ void __launch_bounds__(256)
+chan_scan_kernel(const T* __restrict__ xc, const T* __restrict__ low, int low_ld, const T* __restrict__ wdt, int R, int Rp,
+                 const float* __restrict__ dt_bias, const float* __restrict__ A, const float* __restrict__ Dv,
+                 const T* __restrict__ proj, int ld, int zoff, float* __restrict__ state, const int* __restrict__ slots,
+                 const int* __restrict__ q_start, const int* __restrict__ ctx_len, T* __restrict__ out, int inner, int N,
+                 int nslots, float* __restrict__ ws, float* __restrict__ wa, int chunk_len, int maxchunks) {
+  constexpr float LOG2E = 1.4426950408889634f;
+  constexpr int NP = 4 * NPT;
+  typedef float f32x2_t __attribute__((ext_vector_type(2)));
+  __shared__ __attribute__((aligned(16))) float bc[SC_TB][2][NP];
+  __shared__ __attribute__((aligned(16))) f32x2_t sd[SC_TB][SC_CH];
+  __shared__ float sy[MODE == 1 ? 1 : SC_TB][SC_CH];
+  const int seq = blockIdx.y, c0 = blockIdx.x * SC_CH;
+  int qa = q_start[seq], qlen = q_start[seq + 1] - qa;
+  if (qlen <= 0) return;
+  const bool fresh = ctx_len[seq] - qlen == 0;
+  const int slot = MODE == 0 ? slots[seq] : 0;
+  const bool slot_ok = MODE == 0 ? index_ok(slot, nslots, ERR_SAMPLER_SLOT) : true;
+  float* Sb = state + (size_t)(slot_ok ? slot : 0) * inner * N;
+  int chunk = 0;
+  if (MODE != 0) {
+    chunk = blockIdx.z;
+    if (chunk * chunk_len >= qlen) return;
+    qa += chunk * chunk_len;
+    qlen = min(chunk_len, qlen - chunk * chunk_len);
+    Sb = ws + (size_t)(seq * maxchunks + chunk) * inner * N;
+  }
+  const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6, ql = lane & 15, quad = lane >> 4;
+  // walk role: channel ch, part of its numbers
+  const int cl = threadIdx.x >> 2, part = threadIdx.x & 3, ch = c0 + cl;
+  const bool ch_ok = ch < inner;
+  float S[NPT], a2[NPT];
+  const bool vecn = (N & 3) == 0;
+#pragma unroll
+  for (int j = 0; j < NPT / 4; ++j) {
+    const int n0 = 4 * (part + 4 * j);
+    f32x4_t av = f32x4_t{0.f, 0.f, 0.f, 0.f}, sv = av;
+    if (ch_ok && n0 < N) {
+      const float* ap = A + (size_t)ch * N + n0;
+      const float* sp = Sb + (size_t)ch * N + n0;
+      const bool use = MODE == 2 || (MODE == 0 && !fresh && slot_ok);
+      if (vecn) {
+        av = *reinterpret_cast<const f32x4_t*>(ap);
+        if (use) sv = *reinterpret_cast<const f32x4_t*>(sp);
+      } else {
+#pragma unroll
+        for (int e = 0; e < 4; ++e)
+          if (n0 + e < N) {
+            av[e] = ap[e];
+            if (use) sv[e] = sp[e];
+          }
+      }
+    }
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+      a2[4 * j + e] = av[e];
+      S[4 * j + e] = sv[e];
+    }
+  }
+  // staging role: channel sc of tokens 4 quad + i
+  const int sc = c0 + 16 * wid + ql;
+  const bool sc_ok = sc < inner;
+  const float bias = sc_ok ? dt_bias[sc] : 0.f, dsk = sc_ok ? Dv[sc] : 0.f;
+  const T* wrow = wdt + (size_t)(sc_ok ? sc : 0) * Rp;
+  constexpr int NW = 4;  // matrix fragments kept in registers (R up to 128); the rest is read again per tile
+  bf16x8_t wf[NW];
+  if (sizeof(T) == 2) {
+#pragma unroll
+    for (int k = 0; k < NW; ++k)
+      wf[k] = 32 * k < Rp ? *reinterpret_cast<const bf16x8_t*>(wrow + 32 * k + 8 * quad) : bf16x8_t{0, 0, 0, 0, 0, 0, 0, 0};
+  }
+  float dtsum = 0.f;
+  for (int t0 = 0; t0 < qlen; t0 += SC_TB) {
+    const int nb = min(SC_TB, qlen - t0);
+    // step sizes before softplus
+    float dv[4] = {bias, bias, bias, bias};
+    if (sizeof(T) == 2) {
+      f32x4_t acc = f32x4_t{bias, bias, bias, bias};
+      const T* lrow = low + (size_t)(qa + t0 + (ql < nb ? ql : 0)) * low_ld + 8 * quad;
+      auto frag = [&](int k) {  // (rows are padded to a multiple of 8, so a vector that starts below R lies in its row)
+        return 32 * k + 8 * quad < R ? *reinterpret_cast<const bf16x8_t*>(lrow + 32 * k) : bf16x8_t{0, 0, 0, 0, 0, 0, 0, 0};
+      };
+#pragma unroll
+      for (int k = 0; k < NW; ++k)
+        if (32 * k < Rp) acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(frag(k), wf[k], acc, 0, 0, 0);
+      for (int k = NW; 32 * k < Rp; ++k)
+        acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(frag(k), *reinterpret_cast<const bf16x8_t*>(wrow + 32 * k + 8 * quad),
+                                                      acc, 0, 0, 0);
+#pragma unroll
+      for (int i = 0; i < 4; ++i) dv[i] = acc[i];
+    } else {
+      for (int k = 0; k < R; ++k) {
+        const float w = lds(wrow + k);
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+          const int t = 4 * quad + i;
+          dv[i] = fmaf(lds(low + (size_t)(qa + t0 + (t < nb ? t : 0)) * low_ld + k), w, dv[i]);
+        }
+      }
+    }
+    float xv[4];
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      const int t = 4 * quad + i;
+      xv[i] = (t < nb && sc_ok) ? lds(xc + (size_t)(qa + t0 + t) * inner + sc) : 0.f;
+    }
+    __syncthreads();  // the tile before is consumed
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      const float dt = softplus_f(dv[i]);
+      sd[4 * quad + i][16 * wid + ql] = f32x2_t{dt * LOG2E, dt * xv[i]};
+    }
+    for (int idx = threadIdx.x; idx < nb * 2 * NP; idx += 256) {
+      const int t = idx / (2 * NP), r = idx - t * 2 * NP, n = r & (NP - 1);
+      bc[t][r / NP][n] = n < N ? lds(low + (size_t)(qa + t0 + t) * low_ld + R + (r < NP ? 0 : N) + n) : 0.f;
+    }
+    __syncthreads();
+    for (int t = 0; t < nb; ++t) {
+      const f32x2_t d = sd[t][cl];
+      float y = 0.f;
+#pragma unroll
+      for (int j = 0; j < NPT / 4; ++j) {
+        const f32x4_t b4 = *reinterpret_cast<const f32x4_t*>(&bc[t][0][4 * (part + 4 * j)]);
+#pragma unroll
+        for (int e = 0; e < 4; ++e)
+          S[4 * j + e] = fmaf(__builtin_amdgcn_exp2f(d[0] * a2[4 * j + e]), S[4 * j + e], d[1] * b4[e]);
+        if (MODE != 1) {
+          const f32x4_t c4 = *reinterpret_cast<const f32x4_t*>(&bc[t][1][4 * (part + 4 * j)]);
+#pragma unroll
+          for (int e = 0; e < 4; ++e) y = fmaf(S[4 * j + e], c4[e], y);
+        }
+      }
+      if (MODE == 1) dtsum += d[0];
+      else sy[t][cl] = quad_sum(y);
+    }
+    if (MODE != 1) {
+      __syncthreads();
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        const int t = 4 * quad + i;
+        if (t < nb && sc_ok) {
+          const float zv = lds(proj + (size_t)(qa + t0 + t) * ld + zoff + sc);
+          sts(out + (size_t)(qa + t0 + t) * inner + sc, fmaf(dsk, xv[i], sy[t][16 * wid + ql]) * silu_f(zv));
+        }
+      }
+    }
+  }
+  if (MODE != 2 && slot_ok && ch_ok) {
+#pragma unroll
+    for (int j = 0; j < NPT / 4; ++j) {
+      const int n0 = 4 * (part + 4 * j);
+      if (n0 >= N) continue;
+      float* sp = Sb + (size_t)ch * N + n0;
+      if (vecn) {
+        *reinterpret_cast<f32x4_t*>(sp) = f32x4_t{S[4 * j], S[4 * j + 1], S[4 * j + 2], S[4 * j + 3]};
+      } else {
+#pragma unroll
+        for (int e = 0; e < 4; ++e)
+          if (n0 + e < N) sp[e] = S[4 * j + e];
+      }
+    }
+  }
+  if (MODE == 1 && part == 0 && ch_ok) wa[(size_t)(seq * maxchunks + chunk) * inner + ch] = dtsum;
+}
+
+// ws[seq, c] (chunk c's own contribution) -> the state at the start of chunk c; the slot's state <- the state after the
+// last chunk.  grid (ceil(inner * N / 256), nseq): one thread per state number.
+__global__ void chan_chunk_prefix_kernel(float* __restrict__ state, const int* __restrict__ slots,
+                                         const int* __restrict__ q_start, const int* __restrict__ ctx_len,
+                                         const float* __restrict__ A, float* __restrict__ ws, const float* __restrict__ wa,
+                                         int chunk_len, int maxchunks, int inner, int N, int nslots) {
+  const int seq = blockIdx.y, e = blockIdx.x * 256 + threadIdx.x;
+  const int qlen = q_start[seq + 1] - q_start[seq];
+  if (qlen <= 0 || e >= inner * N) return;
+  const bool fresh = ctx_len[seq] - qlen == 0;
+  const int slot = slots[seq];
+  if (!index_ok(slot, nslots, ERR_SAMPLER_SLOT)) return;
+  float* Sg = state + (size_t)slot * inner * N + e;
+  const int nch = (qlen + chunk_len - 1) / chunk_len, c = e / N;
+  const float a = A[e];
+  float S = fresh ? 0.f : *Sg;
+  float* w = ws + (size_t)seq * maxchunks * inner * N + e;
+  const float* d = wa + (size_t)seq * maxchunks * inner + c;
+  for (int k = 0; k < nch; ++k) {
+    const float u = w[(size_t)k * inner * N];
+    w[(size_t)k * inner * N] = S;
+    S = fmaf(__builtin_amdgcn_exp2f(d[(size_t)k * inner] * a), S, u);
+  }
+  *Sg = S;
+}
+
 }  // namespace grag
 
 using namespace grag;
@@ -333,5 +554,66 @@ GRAG_API hipError_t grag_ssm_scan(const void* xbc, int C, int boff, int coff, co
   DT_DISPATCH(dt, e = (launch_ssm_scan<T, 2>((const T*)xbc, C, boff, coff, (const T*)proj, ld, dtoff, dt_bias, A_log, Dv,
                                              state, slots, q_start, ctx_len, out, nseq, H, G, N, P, nslots, ws, wa,
                                              maxchunks, st));)
+  return e;
+}
+
+GRAG_API int grag_chan_scan_tile() { return SC_CH; }
+GRAG_API int grag_chan_scan_max_state() { return 256; }
+
+template <typename T, int MODE>
+static hipError_t launch_chan_scan(const T* xc, const T* low, int low_ld, const T* wdt, int R, int Rp, const float* dt_bias,
+                                   const float* A, const float* Dv, const T* proj, int ld, int zoff, float* state,
+                                   const int* slots, const int* q_start, const int* ctx_len, T* out, int nseq, int inner,
+                                   int N, int nslots, float* ws, float* wa, int chunk_len, int maxchunks, hipStream_t st) {
+  const dim3 grid((inner + SC_CH - 1) / SC_CH, nseq, MODE == 0 ? 1 : maxchunks);
+#define CHAN_LAUNCH(NPT)                                                                                              \
+  hipLaunchKernelGGL((chan_scan_kernel<T, NPT, MODE>), grid, dim3(256), 0, st, xc, low, low_ld, wdt, R, Rp, dt_bias,  \
+                     A, Dv, proj, ld, zoff, state, slots, q_start, ctx_len, out, inner, N, nslots, ws, wa, chunk_len, \
+                     maxchunks)
+  if (N <= 16) {
+    CHAN_LAUNCH(4);
+  } else if (N <= 32) {
+    CHAN_LAUNCH(8);
+  } else if (N <= 64) {
+    CHAN_LAUNCH(16);
+  } else if (N <= 128) {
+    CHAN_LAUNCH(32);
+  } else {
+    CHAN_LAUNCH(64);
+  }
+#undef CHAN_LAUNCH
+  return hipGetLastError();
+}
+
+// chunk_len 0 (or ws / wa null, or max_q_len <= chunk_len): one pass; else the chunk-parallel passes over ws [nseq *
+// ceil(max_q_len / chunk_len)][inner][N] and wa [nseq * chunks][inner] fp32, chunk_len a multiple of 16.
+GRAG_API hipError_t grag_chan_scan(const void* xc, const void* low, int low_ld, const void* wdt, int R, int Rp,
+                                   const float* dt_bias, const float* A, const float* Dv, const void* proj, int ld,
+                                   int zoff, float* state, const int* slots, const int* q_start, const int* ctx_len,
+                                   void* out, int nseq, int inner, int N, int nslots, int dt, float* ws, float* wa,
+                                   int chunk_len, int max_q_len, hipStream_t st) {
+  if (nseq <= 0 || max_q_len <= 0) return hipSuccess;
+  if (N < 1 || N > 256 || inner < 1 || R < 1 || Rp < R || Rp % 32 || nseq > 65535 || low_ld < R + 2 * N ||
+      (reinterpret_cast<uintptr_t>(A) & 15) || (reinterpret_cast<uintptr_t>(state) & 15))
+    return hipErrorInvalidValue;
+  if (dt == 0 && (low_ld % 8 || (reinterpret_cast<uintptr_t>(low) & 15) || (reinterpret_cast<uintptr_t>(wdt) & 15)))
+    return hipErrorInvalidValue;
+  if (ws == nullptr || wa == nullptr || chunk_len <= 0 || max_q_len <= chunk_len) {
+    DT_DISPATCH(dt, return (launch_chan_scan<T, 0>((const T*)xc, (const T*)low, low_ld, (const T*)wdt, R, Rp, dt_bias, A, Dv,
+                                                   (const T*)proj, ld, zoff, state, slots, q_start, ctx_len, (T*)out, nseq,
+                                                   inner, N, nslots, nullptr, nullptr, 0, 0, st));)
+  }
+  const int maxchunks = (max_q_len + chunk_len - 1) / chunk_len;
+  if (chunk_len % SC_TB || maxchunks > 65535 || (reinterpret_cast<uintptr_t>(ws) & 15)) return hipErrorInvalidValue;
+  hipError_t e;
+  DT_DISPATCH(dt, e = (launch_chan_scan<T, 1>((const T*)xc, (const T*)low, low_ld, (const T*)wdt, R, Rp, dt_bias, A, Dv,
+                                              (const T*)proj, ld, zoff, state, slots, q_start, ctx_len, (T*)out, nseq,
+                                              inner, N, nslots, ws, wa, chunk_len, maxchunks, st));)
+  if (e != hipSuccess) return e;
+  hipLaunchKernelGGL(chan_chunk_prefix_kernel, dim3((unsigned)(((size_t)inner * N + 255) / 256), nseq), dim3(256), 0, st,
+                     state, slots, q_start, ctx_len, A, ws, wa, chunk_len, maxchunks, inner, N, nslots);
+  DT_DISPATCH(dt, e = (launch_chan_scan<T, 2>((const T*)xc, (const T*)low, low_ld, (const T*)wdt, R, Rp, dt_bias, A, Dv,
+                                              (const T*)proj, ld, zoff, state, slots, q_start, ctx_len, (T*)out, nseq,
+                                              inner, N, nslots, ws, wa, chunk_len, maxchunks, st));)
   return e;
 }

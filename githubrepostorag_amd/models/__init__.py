@@ -26,6 +26,10 @@ def build_decoder(cfg, **kw):
         from .pubulix import PubulixModel
 
         return PubulixModel(cfg, **kw)
+    if cfg.arch == "vudivik":
+        from .vudivik import VudivikModel
+
+        return VudivikModel(cfg, **kw)
     from .qwen2 import Qwen2Model
 
     return Qwen2Model(cfg, **kw)

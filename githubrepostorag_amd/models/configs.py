@@ -79,6 +79,16 @@ class EncoderConfig:
 
 
 @dataclass(frozen=True)
+class RopeScaling:
+    """Rotary frequencies by wavelength l: kept below original / high, divided by ``factor`` above original / low, a
+    blend of the two in between, linear in original / l."""
+    factor: float
+    low: float
+    high: float
+    original: float
+
+
+@dataclass(frozen=True)
 class SinkAttnSpec:
     """Softmax attention with a per-head sink, GQA, partial rotary and RMS-normed values."""
     heads: int
@@ -159,6 +169,33 @@ class CappedAttnSpec:
 
 
 @dataclass(frozen=True)
+class NormedAttnSpec:
+    """Softmax attention with biased projections, an RMS norm per query / key head, partial rotary on halves (``scaling``:
+    the stretch of its long wavelengths, see RopeScaling) and a sliding window (0: plain causal) that also sees the
+    sequence's first ``keep_first`` positions."""
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    scale: float
+    window: int
+    keep_first: int
+    rot_dims: int
+    rot_base: float
+    scaling: RopeScaling | None = None
+
+
+@dataclass(frozen=True)
+class SelectiveSSMSpec:
+    """Selective scan with a decay per channel and state number: ``inner`` channels of ``state`` numbers each (fp32),
+    step sizes through ``dt_rank`` numbers per token, a causal convolution of ``taps`` taps in front."""
+    inner: int
+    state: int
+    dt_rank: int
+    taps: int
+
+
+@dataclass(frozen=True)
 class ChunkAttnSpec:
     """Softmax attention inside aligned blocks of ``chunk`` positions (0: plain causal), GQA, partial rotary on
     adjacent pairs, a temperature per head, a sigmoid output gate per head."""
@@ -207,13 +244,16 @@ class MoESpec:
     shared_ff: int
     limit: float | None = None  # clamped units g sigmoid(1.702 g) (u + 1), g = min(gate, limit), u = clamp(up, +-limit)
     table: bool = False  # no router: a [vocab, top] table names every token id's experts, each weighs 1 / top
+    unit: str = "glu"  # "glu": gate and up branches; "relu2": one up branch, squared relu
+    correction: bool = False  # a learned number per logit row joins the scores that choose, not the weights
+    identity: int = 0  # logit rows behind the experts' whose "expert" returns its input
 
 
 @dataclass(frozen=True)
 class MixerSpec:
     kind: str  # "parallel" | "mingru" | "retention" | "attention" | "latent_attention" | "mamba2"
-    left: SinkAttnSpec | None = None
-    right: DecayAttnSpec | None = None
+    left: SinkAttnSpec | NormedAttnSpec | None = None
+    right: DecayAttnSpec | SelectiveSSMSpec | None = None
     left_scale: float = 1.0
     right_scale: float = 1.0
     width: int = 0  # mingru state width
@@ -228,9 +268,18 @@ class GLUSpec:
 
 
 @dataclass(frozen=True)
+class MLPSpec:
+    """One up branch, an activation ("relu2": squared relu), one down matrix."""
+    kind: str  # "dense"
+    ff: int
+    act: str = "relu2"
+
+
+@dataclass(frozen=True)
 class HybridLayerSpec:
     mixer: MixerSpec
-    mlp: GLUSpec | MoESpec | None
+    mlp: GLUSpec | MLPSpec | MoESpec | None
+    weights_of: int | None = None  # this layer runs on that layer's tensors, with a cache and state of its own
 
 
 @dataclass(frozen=True)
@@ -268,11 +317,36 @@ class HybridConfig:
         runs += [(i, 0, False) for i in range(b, n)]
         return runs
 
+    def tensor_layer(self, i: int) -> int:
+        """The layer whose tensors layer i runs on (itself, unless it names another)."""
+        seen = {i}
+        while self.layers[i].weights_of is not None:
+            i = self.layers[i].weights_of
+            if not 0 <= i < len(self.layers) or i in seen:
+                raise ValueError(f"weights_of names no layer with tensors of its own (layer {i})")
+            seen.add(i)
+        return i
+
     def to_dict(self):
         return asdict(self)
 
     def param_count(self) -> int:
         H = self.hidden_size
+        if self.arch == "vudivik":
+            n = 2 * self.vocab_size * H + H
+            for L in self.layers:
+                if L.weights_of is not None:
+                    continue
+                a, r, f = L.mixer.left, L.mixer.right, L.mlp
+                qkv = a.heads * a.dim + a.kv_heads * (a.dim + a.vdim)
+                n += H + (H + 1) * qkv + 2 * a.dim + a.heads * a.vdim * H + H
+                n += 2 * r.inner * H + r.inner * (r.taps + 1) + (r.dt_rank + 2 * r.state) * r.inner + r.inner * r.dt_rank
+                n += r.inner * (r.state + 2) + r.inner * H + H
+                if isinstance(f, MLPSpec):
+                    n += H + 2 * H * f.ff
+                elif f is not None:
+                    n += H + f.experts * 2 * H * f.ff + (f.experts + f.identity) * (H + 1)
+            return n
         if self.arch == "pubulix":
             n = 2 * self.vocab_size * H + 1
             for L in self.layers:
@@ -670,6 +744,100 @@ def pubulix_config(name: str, vocab: int, width: int, pattern: str, *, heads: in
                         residual_mult=residual_mult, logit_softcap=logit_softcap, conv_taps=taps)
 
 
+def vudivik_config_from_dict(d: dict, name: str = "vudivik") -> HybridConfig:
+    """The Vudivik design's config.json: a layer list of "parallel" mixers (windowed GQA attention that keeps the first
+    tokens, beside a selective scan), each with an optional squared-relu feed-forward, dense or a mixture of experts
+    some of which are the identity; a layer may run on an earlier or later layer's tensors.  Every size and constant is
+    read from it."""
+    layers = []
+    for i, e in enumerate(d["layers"]):
+        if e["type"] != "parallel":
+            raise ValueError(f"unknown mixer type {e['type']!r}")
+        l, r = e["mixer"]["left"], e["mixer"]["right"]
+        rot, mask = l.get("rot") or {"dims": 0, "base": 1.0}, l.get("mask") or {}
+        sc = rot.get("scaling")
+        dim = int(l["dim"])
+        left = NormedAttnSpec(int(l["heads"]), int(l.get("kv_heads", l["heads"])), dim, int(l.get("vdim", dim)),
+                              float(l["scale"]), int(mask.get("size") or 0), int(mask.get("keep_first") or 0),
+                              int(rot["dims"]), float(rot.get("base", 1.0)),
+                              None if not sc else RopeScaling(float(sc["factor"]), float(sc["low"]), float(sc["high"]),
+                                                              float(sc["original"])))
+        if (left.heads % left.kv_heads or left.rot_dims % 2 or left.rot_dims > left.dim or left.window < 0
+                or left.keep_first < 0):
+            raise ValueError(f"bad attention sizes {l}")
+        right = SelectiveSSMSpec(int(r["inner"]), int(r["state"]), int(r["dt_rank"]), int(r["conv"]))
+        if min(right.inner, right.state, right.dt_rank, right.taps) < 1:
+            raise ValueError(f"bad selective-scan sizes {r}")
+        f = e.get("mlp")
+        if f is None:
+            mlp = None
+        elif f.get("kind", "dense") == "dense":
+            mlp = MLPSpec("dense", int(f["ff"]))
+        elif f["kind"] == "moe":
+            rt = f["router"]
+            mlp = MoESpec("moe", int(f["expert"]["ff"]), int(rt["experts"]), int(rt["top"]), 1, 1, 0, unit="relu2",
+                          correction=True, identity=int(rt.get("identity") or 0))
+            if mlp.experts < 1 or mlp.identity < 0 or not 1 <= mlp.top <= mlp.experts + mlp.identity:
+                raise ValueError(f"bad router sizes {rt}")
+        else:
+            raise ValueError(f"unknown feed-forward kind {f['kind']!r}")
+        src = e.get("weights_of")
+        layers.append(HybridLayerSpec(MixerSpec("parallel", left, right), mlp, None if src is None else int(src)))
+    cfg = HybridConfig(name, int(d["vocab"]), int(d["width"]), float(d["norm"]["eps"]), tuple(layers), arch="vudivik",
+                       residual_mult=float(d.get("residual_mult", 1.0)))
+    for i, L in enumerate(layers):
+        o = cfg.layers[cfg.tensor_layer(i)]
+        if (o.mixer, o.mlp) != (L.mixer, L.mlp):
+            raise ValueError(f"layer {i} differs from layer {L.weights_of}, whose tensors it uses")
+    return cfg
+
+
+def vudivik_config_to_dict(cfg: HybridConfig) -> dict:
+    """Back to the config.json form (checkpoint export, tests)."""
+    layers = []
+    for L in cfg.layers:
+        a, r, f = L.mixer.left, L.mixer.right, L.mlp
+        rot = {"dims": a.rot_dims, "base": a.rot_base}
+        if a.scaling is not None:
+            rot["scaling"] = asdict(a.scaling)
+        if f is None:
+            mlp = None
+        elif isinstance(f, MLPSpec):
+            mlp = {"kind": "dense", "ff": f.ff}
+        else:
+            mlp = {"kind": "moe", "expert": {"ff": f.ff},
+                   "router": {"experts": f.experts, "identity": f.identity, "top": f.top}}
+        e = {"type": "parallel", "mlp": mlp, "mixer": {
+            "left": {"heads": a.heads, "kv_heads": a.kv_heads, "dim": a.dim, "vdim": a.vdim, "scale": a.scale,
+                     "mask": {"size": a.window, "keep_first": a.keep_first}, "rot": rot},
+            "right": {"inner": r.inner, "state": r.state, "dt_rank": r.dt_rank, "conv": r.taps}}}
+        if L.weights_of is not None:
+            e["weights_of"] = L.weights_of
+        layers.append(e)
+    return {"architecture": "Vudivik", "vocab": cfg.vocab_size, "width": cfg.hidden_size, "norm": {"eps": cfg.norm_eps},
+            "residual_mult": cfg.residual_mult, "layers": layers}
+
+
+def vudivik_config(name: str, vocab: int, width: int, pattern: str, *, heads: int, kv_heads: int, dim: int, ff: int,
+                   window: int = 1024, keep_first: int = 16, vdim: int | None = None, rot_dims: int | None = None,
+                   scaling=RopeScaling(8.0, 1.0, 4.0, 8192.0), inner: int | None = None, state: int = 16,
+                   dt_rank: int | None = None, taps: int = 4, experts: int = 16, identity: int = 2, top: int = 4,
+                   expert_ff: int | None = None, residual_mult: float = 0.7, eps: float = 1e-6,
+                   shared: dict | None = None) -> HybridConfig:
+    """A regular Vudivik stack for benches and plumbing tests.  ``pattern``: one letter per layer, d = dense feed-forward,
+    m = mixture of experts, n = no feed-forward; ``shared`` {i: j}: layer i runs on layer j's tensors."""
+    inner = inner or 2 * width
+    left = NormedAttnSpec(heads, kv_heads, dim, vdim or dim, dim ** -0.5, window, keep_first,
+                          dim if rot_dims is None else rot_dims, 5e5, scaling)
+    mixer = MixerSpec("parallel", left, SelectiveSSMSpec(inner, state, dt_rank or -(-width // 16), taps))
+    mlps = {"d": MLPSpec("dense", ff), "n": None,
+            "m": MoESpec("moe", expert_ff or -(-ff // top), experts, top, 1, 1, 0, unit="relu2", correction=True,
+                         identity=identity)}
+    return HybridConfig(name, vocab, width, eps, tuple(HybridLayerSpec(mixer, mlps[c], (shared or {}).get(i))
+                                                       for i, c in enumerate(pattern)),
+                        arch="vudivik", residual_mult=residual_mult)
+
+
 def zofesun_config(name: str, vocab: int, width: int, n_layers: int, *, heads: int, kv_heads: int, dim: int,
                    vdim: int, lin_heads: int, lin_dim: int, lin_vdim: int, ff: int, mingru_every: int = 0,
                    rot_dims: int | None = None, rot_base: float = 10000.0, loop=(0, 0, 1), limit: float = 7.0,
@@ -723,6 +891,13 @@ HYBRIDS = {
                                  lat_heads=12, kv_rank=192, rot_dim=64, lat_window=2048, experts=16, top=4, ff=2240),
     "pubulix-7b": pubulix_config("pubulix-7b", 32768, 3584, "alas", heads=28, kv_heads=4, dim=128, window=1024,
                                  lat_heads=28, kv_rank=192, rot_dim=64, lat_window=2048, experts=16, top=4, ff=4736),
+    # Vudivik: a plumbing-test size and two bench sizes with the layer shapes of a 1.5B / 7B decoder (squared-relu
+    # feed-forwards as wide as the dense decoders' gate; the experts' active width top * ff equals it)
+    "vudivik-tiny": vudivik_config("vudivik-tiny", 320, 96, "dmnd", heads=4, kv_heads=2, dim=16, vdim=24, ff=160, window=9,
+                                   keep_first=3, rot_dims=8, scaling=RopeScaling(4.0, 1.0, 4.0, 64.0), inner=72, state=6,
+                                   dt_rank=7, taps=3, experts=6, identity=2, top=3, expert_ff=40, shared={3: 0}),
+    "vudivik-1b": vudivik_config("vudivik-1b", 32768, 1536, "dmdmdmdm", heads=12, kv_heads=2, dim=128, ff=8960),
+    "vudivik-7b": vudivik_config("vudivik-7b", 32768, 3584, "dmdm", heads=28, kv_heads=4, dim=128, ff=18944),
 }
 
 
@@ -739,6 +914,8 @@ def config_from_dir(path) -> DecoderConfig | HybridConfig:
         return leripel_config_from_dict(d, Path(path).name or "leripel")
     if arch == "pubulix":
         return pubulix_config_from_dict(d, Path(path).name or "pubulix")
+    if arch == "vudivik":
+        return vudivik_config_from_dict(d, Path(path).name or "vudivik")
     mt = str(d.get("model_type", "")).lower()
     if mt == "gpt2":
         return DecoderConfig(Path(path).name, d["vocab_size"], d["n_embd"], d.get("n_inner") or 4 * d["n_embd"],

@@ -81,9 +81,10 @@ _SIGS = {
     "grag_err_alloc": [P],
     "grag_embed_f32": [P, P, P, I, I, I, I, F, P],
     "grag_dyt_residual": [P, F, P, P, P, P, P, F, P, P, P, I, I, I, P],
-    "grag_rope_vnorm_store": [P, I, I, I, I, P, P, I, P, P, P, P, I, I, I, I, I, I, I, ctypes.c_long, F, I, I, P],
-    "grag_sink_attn_prefill": [P, P, P, P, I, P, I, P, P, P, I, I, I, I, I, I, I, F, F, I, I, I, P, P, I, I, I, F, P],
-    "grag_sink_attn_decode": [P, P, P, P, I, P, I, P, P, I, I, I, I, I, I, F, F, I, I, I, I, P, P, I, P, P, I, I, I, F, P],
+    "grag_rope_vnorm_store": [P, I, I, I, I, P, P, I, P, P, P, P, I, I, I, I, I, I, I, ctypes.c_long, F, I, I, P, P, P, P],
+    "grag_sink_attn_prefill": [P, P, P, P, I, P, I, P, P, P, I, I, I, I, I, I, I, F, F, I, I, I, P, P, I, I, I, F, I, P],
+    "grag_sink_attn_decode": [P, P, P, P, I, P, I, P, P, I, I, I, I, I, I, F, F, I, I, I, I, P, P, I, P, P, I, I, I, F, I, P],
+    "grag_relu2": [P, I64, I, P],
     "grag_decay_attn_scan": [P, I, I, I, I, P, P, P, P, P, P, I, I, I, I, I, I, P, I, I, P, P, I, I, F, P],
     "grag_decay_attn_chunk": [],
     "grag_mingru_chunk": [],
@@ -105,12 +106,17 @@ _SIGS = {
     "grag_causal_conv": [P, I, I, I, I, P, P, P, P, P, P, P, I, I, I, I, I, P],
     "grag_ssm_chunk": [],
     "grag_ssm_scan": [P, I, I, I, P, I, I, P, P, P, P, P, P, P, P, I, I, I, I, I, I, I, P, P, I, P],
+    "grag_chan_scan_tile": [],
+    "grag_chan_scan_max_state": [],
+    "grag_chan_scan": [P, P, I, P, I, I, P, P, P, P, I, I, P, P, P, P, P, I, I, I, I, I, P, P, I, I, P],
     "grag_moe_max_rows": [],
     "grag_moe_max_top": [],
-    "grag_moe_route": [P, I, P, I, I, I, I, I, I, P, P, P, I, I, P],
+    "grag_moe_route": [P, I, P, I, I, I, I, I, I, P, P, P, I, I, P, I, P, P],
     "grag_moe_align": [P, I, I, P, P, P],
     "grag_moe_gemm": [P, I, P, P, P, I, I, I, I, I, P, I, I, I, F, F, F, P, I, P],
     "grag_moe_table_route": [P, P, I, I, I, P, P, I, P],
+    "grag_postnorm_max_width": [],
+    "grag_postnorm_residual": [P, P, P, P, P, F, P, P, I, P, P, F, F, P, P, I, I, I, P],
     "grag_residual_rmsnorm": [P, F, P, P, P, P, P, I, P, F, P, P, I, I, I, I, P, I, P, F, P],
 }
 

@@ -149,30 +149,48 @@ def softmax_scale(head_dim: int) -> float:
 
 
 # ---------------------------------------------------------------------------------------------- partial rotary + value norm
-def rope_table(max_pos: int, rot_dims: int, base: float, device=None) -> torch.Tensor:
+def rope_table(max_pos: int, rot_dims: int, base: float, device=None, scaling=None) -> torch.Tensor:
     """[max_pos, rot_dims] fp32: cos(p f_i) in [:rot_dims/2], sin in [rot_dims/2:], f_i = base^(-2i/rot_dims);
-    angles formed in float64 and rounded once."""
+    angles formed in float64 and rounded once.  ``scaling`` (factor, low, high, original as attributes): frequencies
+    are blended by their wavelength l = 2 pi / f between f (l < original / high) and f / factor (l > original / low),
+    the share of f being (original / l - low) / (high - low) in between."""
     i = torch.arange(rot_dims // 2, dtype=torch.float64)
-    f = torch.outer(torch.arange(max_pos, dtype=torch.float64), torch.as_tensor(base, dtype=torch.float64) ** (-2.0 * i / max(1, rot_dims)))
+    fr = torch.as_tensor(base, dtype=torch.float64) ** (-2.0 * i / max(1, rot_dims))
+    if scaling is not None:
+        turns = scaling.original * fr / (2.0 * math.pi)  # original / wavelength
+        mid = (turns - scaling.low) / (scaling.high - scaling.low) if scaling.high != scaling.low else torch.zeros_like(fr)
+        share = torch.where(turns > scaling.high, torch.ones_like(fr),
+                            torch.where(turns < scaling.low, torch.zeros_like(fr), mid))
+        fr = (1.0 - share) * fr / scaling.factor + share * fr
+    f = torch.outer(torch.arange(max_pos, dtype=torch.float64), fr)
     return torch.cat([f.cos(), f.sin()], dim=-1).float().to(device)
 
 
 def rope_vnorm_store(proj: torch.Tensor, qoff: int, koff: int, voff: int, positions: torch.Tensor,
                      table: torch.Tensor, slot_mapping: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor,
                      H: int, G: int, d: int, vd: int, rot_dims: int, eps: float, interleaved: bool = False,
-                     vnorm: bool = True) -> torch.Tensor:
+                     vnorm: bool = True, bias: torch.Tensor | None = None, qw: torch.Tensor | None = None,
+                     kw: torch.Tensor | None = None) -> torch.Tensor:
     """From a fused projection ``proj`` [T, ld] (q heads at column qoff, k at koff, v at voff): rotate the first
     ``rot_dims`` dims of every q / k head (dim i paired with i + rot_dims/2; ``interleaved``: dim 2i with 2i + 1,
     pair i turned by the table's angle i), divide every v head by its root mean square (fp32; ``vnorm`` False: the
     values as they are), store k / v into the paged caches k_cache [blocks, G, BS, d] / v_cache [blocks, G, BS, vd]
-    at ``slot_mapping`` (-1: not stored) and return q [T, H, d]."""
+    at ``slot_mapping`` (-1: not stored) and return q [T, H, d].  ``bias`` [>= all columns used] fp32 is added to the
+    projection first, by column; ``qw`` / ``kw`` [d] fp32: every q / k head is divided by its root mean square (with
+    ``eps``) and multiplied by them before the rotation.  All of it in fp32; the results are rounded once."""
     T = proj.shape[0]
     BS = k_cache.shape[2]
     if not proj.is_cuda:
         x = proj.float()
+        if bias is not None:
+            x = x[:, :bias.numel()] + bias.float()
         q = x[:, qoff:qoff + H * d].reshape(T, H, d).clone()
         k = x[:, koff:koff + G * d].reshape(T, G, d).clone()
         v = x[:, voff:voff + G * vd].reshape(T, G, vd)
+        if qw is not None:
+            q = q / torch.sqrt(q.pow(2).mean(-1, keepdim=True) + eps) * qw.float()
+        if kw is not None:
+            k = k / torch.sqrt(k.pow(2).mean(-1, keepdim=True) + eps) * kw.float()
         if rot_dims:
             h2 = rot_dims // 2
             cs = table[positions.long()]
@@ -194,11 +212,14 @@ def rope_vnorm_store(proj: torch.Tensor, qoff: int, koff: int, voff: int, positi
         v_cache[sl // BS, :, sl % BS] = v[ok].to(v_cache.dtype)
         return q.to(proj.dtype)
     assert proj.stride(1) == 1 and k_cache.dtype == proj.dtype and v_cache.dtype == proj.dtype
+    assert bias is None or (bias.dtype == torch.float32 and bias.is_contiguous()
+                            and bias.numel() >= max(qoff + H * d, koff + G * d, voff + G * vd))
+    assert all(w is None or (w.dtype == torch.float32 and w.numel() == d) for w in (qw, kw))
     q = torch.empty(T, H, d, dtype=proj.dtype, device=proj.device)
     call("grag_rope_vnorm_store", ptr(proj), proj.stride(0), qoff, koff, voff, ptr(positions), ptr(table),
          0 if table is None else table.shape[0], ptr(slot_mapping), ptr(q), ptr(k_cache), ptr(v_cache), T, H, G, d, vd, rot_dims, BS,
          k_cache.shape[0] * BS, float(eps), 0 if proj.dtype == torch.bfloat16 else 1,
-         (1 if interleaved else 0) | (0 if vnorm else 2))
+         (1 if interleaved else 0) | (0 if vnorm else 2), ptr(bias), ptr(qw), ptr(kw))
     return q
 
 
@@ -342,4 +363,13 @@ def tanh_cap_(x: torch.Tensor, cap: float) -> torch.Tensor:
         return x
     assert x.dim() == 2 and x.stride(1) == 1
     call("grag_tanh_cap", ptr(x), x.stride(0), x.shape[0], x.shape[1], float(cap), 0 if x.dtype == torch.bfloat16 else 1)
+    return x
+
+
+def relu2_(x: torch.Tensor) -> torch.Tensor:
+    """In place: x <- max(x, 0)^2, evaluated in fp32."""
+    if not x.is_cuda:
+        return x.copy_(x.float().clamp_min(0.0).pow(2).to(x.dtype))
+    assert x.is_contiguous()
+    call("grag_relu2", ptr(x), x.numel(), 0 if x.dtype == torch.bfloat16 else 1)
     return x

@@ -16,14 +16,20 @@ def _dt(t: torch.Tensor) -> int:
     return 0 if t.dtype == torch.bfloat16 else 1
 
 
-def moe_route(h: torch.Tensor, wr: torch.Tensor, E: int, top: int, groups: int = 1, keep: int = 1):
+def moe_route(h: torch.Tensor, wr: torch.Tensor, E: int, top: int, groups: int = 1, keep: int = 1,
+              corr: torch.Tensor | None = None, identity: int = 0):
     """h [T, W]; ``wr`` [R, W] fp32 with the experts' router rows first (R = E, or E + 1 when a last row holds the
     shared expert's gate).  Scores s = softmax of the E logits.  The experts form ``groups`` equal groups of
     neighbours; a group's score is its best expert's, and only experts of the ``keep`` best groups can be chosen.
     Returns (ids [T, top] int32: the chosen experts by falling score, wts [T, top] fp32: their scores as they are,
-    gate [T] fp32 = sigmoid of the extra row's logit, or None)."""
+    gate [T] fp32 = sigmoid of the extra row's logit, or None).
+    ``corr`` [E] fp32 joins the scores for the choice only.  ``identity``: the last that many of the E rows are
+    identity experts, whose output is the token itself: their ids (>= E - identity) name no expert, their entries of
+    wts are 0, and the third result is instead idw [T] fp32, the sum of their weights."""
     T, W = h.shape
     R = wr.shape[0]
+    if identity and (R != E or not 0 < identity <= E):
+        raise ValueError("identity experts are the last of the router's rows")
     if E % groups or not 1 <= keep <= groups or not 1 <= top <= E or R not in (E, E + 1):
         raise ValueError("bad router sizes")
     if not h.is_cuda:
@@ -32,9 +38,13 @@ def moe_route(h: torch.Tensor, wr: torch.Tensor, E: int, top: int, groups: int =
         gs = s.view(T, groups, E // groups).amax(-1)
         open_g = torch.zeros(T, groups, dtype=torch.bool)
         open_g.scatter_(1, gs.topk(keep, dim=-1).indices, True)
-        masked = s.masked_fill(~open_g.repeat_interleave(E // groups, dim=1), -1.0)
-        wts, ids = masked.topk(top, dim=-1)
-        wts = wts.clamp_min(0.0)
+        closed = ~open_g.repeat_interleave(E // groups, dim=1)
+        pick = (s if corr is None else s + corr.float()).masked_fill(closed, -float("inf"))
+        ids = pick.sort(dim=-1, descending=True, stable=True).indices[:, :top]
+        wts = s.masked_fill(closed, 0.0).gather(1, ids)
+        if identity:
+            free = ids >= E - identity
+            return ids.to(torch.int32), wts.masked_fill(free, 0.0), (wts * free).sum(-1)
         return ids.to(torch.int32), wts.contiguous(), (torch.sigmoid(z[:, E]) if R > E else None)
     if R > lib().grag_moe_max_rows() or top > lib().grag_moe_max_top():
         raise ValueError(f"the router kernel holds {lib().grag_moe_max_rows()} logit rows and {lib().grag_moe_max_top()} choices")
@@ -42,9 +52,11 @@ def moe_route(h: torch.Tensor, wr: torch.Tensor, E: int, top: int, groups: int =
     ids = torch.empty(T, top, dtype=torch.int32, device=h.device)
     wts = torch.empty(T, top, dtype=torch.float32, device=h.device)
     gate = torch.empty(T, dtype=torch.float32, device=h.device) if R > E else None
+    idw = torch.empty(T, dtype=torch.float32, device=h.device) if identity else None
+    assert corr is None or (corr.dtype == torch.float32 and corr.numel() == E and corr.is_contiguous())
     call("grag_moe_route", ptr(h), h.stride(0), ptr(wr), W, E, R, top, groups, keep, ptr(ids), ptr(wts), ptr(gate), T,
-         _dt(h))
-    return ids, wts, gate
+         _dt(h), ptr(corr), identity, ptr(idw))
+    return ids, wts, idw if identity else gate
 
 
 def moe_table_route(token_ids: torch.Tensor, table: torch.Tensor):
@@ -64,22 +76,30 @@ def moe_table_route(token_ids: torch.Tensor, table: torch.Tensor):
 
 
 def moe_experts(h: torch.Tensor, ids: torch.Tensor, wgu: torch.Tensor, wd: torch.Tensor,
-                limit: float | None = None, alpha: float = 1.0, shift: float = 0.0) -> torch.Tensor:
+                limit: float | None = None, alpha: float = 1.0, shift: float = 0.0,
+                unit: str = "glu") -> torch.Tensor:
     """The chosen experts' outputs, unweighted: h [T, W], ids [T, top] int32, ``wgu`` [E, 2F, W] (every expert's gate
     rows, then its up rows), ``wd`` [E, W, F] -> [T, top, W] with out[t, k] = wd[e] (silu(gate_e h_t) * (up_e h_t)),
     e = ids[t, k].  With ``limit`` / ``alpha`` / ``shift`` the unit is g sigmoid(alpha g) (u + shift) with
-    g = min(gate, limit), u = clamp(up, -limit, limit) (``limit`` None: no clamp)."""
+    g = min(gate, limit), u = clamp(up, -limit, limit) (``limit`` None: no clamp).  ``unit`` "relu2": one branch,
+    ``wgu`` [E, F, W], out[t, k] = wd[e] max(up_e h_t, 0)^2.  A pair whose id names no expert (>= E or negative: an
+    identity expert's) is left out; its row of the result is undefined on the device."""
     T, W = h.shape
     top = ids.shape[1]
     E, F2, _ = wgu.shape
-    F = F2 // 2
+    F = F2 if unit == "relu2" else F2 // 2
     if not h.is_cuda:
         x = h.float()
         out = torch.zeros(T, top, W)
         for t in range(T):
             for k in range(top):
                 e = int(ids[t, k])
+                if not 0 <= e < E:
+                    continue
                 gu = wgu[e].float() @ x[t]
+                if unit == "relu2":
+                    out[t, k] = wd[e].float() @ gu.clamp_min(0.0).pow(2).to(h.dtype).float()
+                    continue
                 g, u = gu[:F], gu[F:]
                 if limit is not None:
                     g, u = g.clamp(max=limit), u.clamp(-limit, limit)
@@ -94,7 +114,8 @@ def moe_experts(h: torch.Tensor, ids: torch.Tensor, wgu: torch.Tensor, wd: torch
     call("grag_moe_align", ptr(ids), n, E, ptr(offs), ptr(order))
     act = torch.empty(n, F, dtype=h.dtype, device=h.device)
     lim = float("inf") if limit is None else float(limit)
-    call("grag_moe_gemm", ptr(h), h.stride(0), ptr(wgu), ptr(offs), ptr(order), n, E, top, F, W, ptr(act), F, 1, _dt(h),
+    call("grag_moe_gemm", ptr(h), h.stride(0), ptr(wgu), ptr(offs), ptr(order), n, E, top, F, W, ptr(act), F,
+         3 if unit == "relu2" else 1, _dt(h),
          lim, float(alpha), float(shift), None, 0)
     out = torch.empty(T, top, W, dtype=h.dtype, device=h.device)
     call("grag_moe_gemm", ptr(act), F, ptr(wd), ptr(offs), ptr(order), n, E, top, W, F, ptr(out), W, 0, _dt(h),

@@ -277,3 +277,47 @@ def residual_rmsnorm(x: torch.Tensor, a: torch.Tensor | None = None, b: torch.Te
          0 if out_dtype == torch.bfloat16 else 1, ptr(gate), 0 if gate is None else gate.stride(0), ptr(gbias),
          float(mult))
     return out
+
+
+# ---------------------------------------------------------------------------------------------- post-norm boundary
+def postnorm_residual(x: torch.Tensor, a: torch.Tensor | None = None, wa: torch.Tensor | None = None,
+                      b: torch.Tensor | None = None, wb: torch.Tensor | None = None, bscale: float = 1.0,
+                      e: torch.Tensor | None = None, ecoef: torch.Tensor | None = None,
+                      idw: torch.Tensor | None = None, w: torch.Tensor | None = None, eps: float = 1e-6,
+                      mult: float = 1.0, wn: torch.Tensor | None = None, out_dtype=torch.bfloat16) -> torch.Tensor:
+    """One pass over the fp32 residual ``x`` [T, H] (updated in place) at the boundary of a sublayer whose OUTPUT is
+    normed: with unit(v) = v / sqrt(mean(v^2) + eps),
+        y = bscale * (unit(a) * wa + unit(b) * wb)             with ``wa`` [H] fp32: mixers side by side, else
+        y = a + sum_k ecoef[t, k] e[t, k] + idw[t] x[t]        every addend optional, pairs of weight 0 are not read;
+        x <- x + mult * unit(y) * w                            (``w`` None: x stays as it is).
+    Returns unit(x) * wn, or x itself without ``wn``, in ``out_dtype``: the next sublayer's input."""
+    assert x.dtype == torch.float32 and x.is_contiguous() and x.dim() == 2
+    T, H = x.shape
+    K = 0 if e is None else e.shape[1]
+    if not _on_gpu(x):
+        unit = lambda v: v / torch.sqrt(v.pow(2).mean(-1, keepdim=True) + eps)
+        if w is not None:
+            if wa is not None:
+                y = unit(a.float()) * wa.float()
+                if b is not None:
+                    y = y + unit(b.float()) * wb.float()
+                y = y * bscale
+            else:
+                y = torch.zeros_like(x) if a is None else a.float().clone()
+                if e is not None:
+                    y += (e.float() * ecoef.float()[:, :, None]).sum(1)
+                if idw is not None:
+                    y += idw.float()[:, None] * x
+            x += mult * unit(y) * w.float()
+        return (x if wn is None else unit(x) * wn.float()).to(out_dtype, copy=True)
+    for t in (a, b):
+        assert t is None or (t.dtype == out_dtype and t.is_contiguous() and t.shape == (T, H))
+    for t in (wa, wb, w, wn):
+        assert t is None or (t.dtype == torch.float32 and t.is_contiguous() and t.numel() == H)
+    assert e is None or (e.dtype == out_dtype and e.is_contiguous() and e.shape == (T, K, H)
+                         and ecoef.dtype == torch.float32 and ecoef.is_contiguous() and ecoef.shape == (T, K))
+    assert idw is None or (idw.dtype == torch.float32 and idw.is_contiguous() and idw.numel() == T)
+    out = torch.empty(T, H, dtype=out_dtype, device=x.device)
+    call("grag_postnorm_residual", ptr(x), ptr(a), ptr(wa), ptr(b), ptr(wb), float(bscale), ptr(e), ptr(ecoef), K, ptr(idw),
+         ptr(w), float(eps), float(mult), ptr(wn), ptr(out), T, H, 0 if out_dtype == torch.bfloat16 else 1)
+    return out

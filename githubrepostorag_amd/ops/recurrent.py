@@ -254,3 +254,78 @@ def _ssm_scan_cpu(xbc, dtraw, dt_bias, a_log, skip, state, m, H, G, N, P, out):
             S = decay[a + t, :, None, None] * S + (dt[a + t, :, None] * B[t])[:, :, None] * x[t][:, None, :]
             out[a + t] = (torch.einsum("hnp,hn->hp", S, Cm[t]) + skip.float()[:, None] * x[t]).reshape(-1)
         state[sl[s]] = S
+
+
+# ---------------------------------------------------------------------------------------------- per-channel scan
+CHAN_SCAN_WGS = 1024  # workgroups (64 channels x one sequence x one chunk) that a portion is cut for
+
+
+def _chan_chunk(nseq: int, max_q: int, inner: int) -> int:
+    """Chunk length of the per-channel scan (0: one pass).  The chunked form does the recurrence twice, so a step with
+    enough (channel tile, sequence) workgroups of its own stays whole; others get the longest chunks that fill the chip."""
+    tiles = nseq * -(-inner // 64)
+    if max_q <= 64 or 2 * tiles >= CHAN_SCAN_WGS:
+        return 0
+    for c in (256, 128):
+        if max_q > 2 * c and tiles * -(-max_q // c) >= CHAN_SCAN_WGS:
+            return c
+    return 64
+
+
+def pad_step_matrix(w: torch.Tensor) -> torch.Tensor:
+    """Columns padded with zeros to a multiple of 32: the form selective_scan reads its step-size matrix in."""
+    return torch.nn.functional.pad(w, (0, -w.shape[1] % 32))
+
+
+def selective_scan(xc: torch.Tensor, low: torch.Tensor, wdt: torch.Tensor, R: int, dt_bias: torch.Tensor,
+                   A: torch.Tensor, skip: torch.Tensor, proj: torch.Tensor, zoff: int, state: torch.Tensor,
+                   meta: AttnMetadata) -> torch.Tensor:
+    """Selective scan with a decay per channel and state number.  ``xc`` [T, inner] (the convolution's output); ``low``
+    [T, >= R + 2N] holds per token R step-size numbers | B (N) | C (N); ``wdt`` [inner, R padded to a multiple of 32]
+    (pad_step_matrix); ``A`` [inner, N] fp32.  Per channel c, in fp32: dt = softplus(wdt_c low + dt_bias_c),
+    S_n <- exp(dt A[c, n]) S_n + dt x_c B_n (state [slots, inner, N]), y = sum_n S_n C_n + skip_c x_c.  Returns
+    y * silu(z) [T, inner] in xc's dtype, z = columns zoff .. zoff + inner of ``proj``."""
+    T, inner = xc.shape
+    N = A.shape[1]
+    out = torch.empty(T, inner, dtype=xc.dtype, device=xc.device)
+    for m, r0, r1 in _parts(meta):
+        if r1 <= r0:
+            continue
+        if not xc.is_cuda:
+            _selective_scan_cpu(xc[r0:r1].float(), low[r0:r1].float(), wdt[:, :R].float(), dt_bias, A, skip,
+                                proj[r0:r1, zoff:zoff + inner].float(), state, m, out[r0:r1])
+            continue
+        assert xc.is_contiguous() and low.is_contiguous() and wdt.is_contiguous() and proj.stride(1) == 1
+        assert xc.dtype == low.dtype == wdt.dtype == proj.dtype and wdt.shape[0] == inner and low.shape[1] >= R + 2 * N
+        assert state.dtype == torch.float32 and state.is_contiguous() and state.shape[1:] == (inner, N)
+        assert all(t.dtype == torch.float32 and t.is_contiguous() for t in (A, dt_bias, skip)) and A.shape[0] == inner
+        assert dt_bias.numel() == inner and skip.numel() == inner and zoff + inner <= proj.shape[1]
+        if N > lib().grag_chan_scan_max_state():
+            raise ValueError(f"the scan kernel holds {lib().grag_chan_scan_max_state()} state numbers per channel")
+        chunk, ws, wa = _chan_chunk(m.num_seqs, m.max_q_len, inner), None, None
+        if chunk:
+            nch = m.num_seqs * -(-m.max_q_len // chunk)
+            ws = torch.empty(nch * inner * N, dtype=torch.float32, device=xc.device)
+            wa = torch.empty(nch * inner, dtype=torch.float32, device=xc.device)
+        call("grag_chan_scan", ptr(xc[r0:r1]), ptr(low[r0:r1]), low.shape[1], ptr(wdt), R, wdt.shape[1], ptr(dt_bias),
+             ptr(A), ptr(skip), ptr(proj[r0:r1]), proj.stride(0), zoff, ptr(state), ptr(m.state_slots), ptr(m.q_start),
+             ptr(m.ctx_len), ptr(out[r0:r1]), m.num_seqs, inner, N, state.shape[0], _dt(xc), ptr(ws), ptr(wa), chunk,
+             m.max_q_len)
+    return out
+
+
+def _selective_scan_cpu(x, low, wdt, dt_bias, A, skip, z, state, m, out):
+    R, N = wdt.shape[1], A.shape[1]
+    qs, cl, sl = m.q_start.tolist(), m.ctx_len.tolist(), m.state_slots.tolist()
+    dt = torch.nn.functional.softplus(low[:, :R] @ wdt.T + dt_bias.float(), threshold=20.0)
+    B, C = low[:, R:R + N], low[:, R + N:R + 2 * N]
+    g = torch.nn.functional.silu(z)
+    for s in range(m.num_seqs):
+        a, e = qs[s], qs[s + 1]
+        if e <= a:
+            continue
+        S = torch.zeros_like(A) if cl[s] - (e - a) == 0 else state[sl[s]].clone()
+        for t in range(a, e):
+            S = torch.exp(dt[t, :, None] * A) * S + (dt[t] * x[t])[:, None] * B[t]
+            out[t] = ((S @ C[t] + skip.float() * x[t]) * g[t]).to(out.dtype)
+        state[sl[s]] = S
