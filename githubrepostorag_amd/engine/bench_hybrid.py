@@ -1,4 +1,4 @@
-"""``bench.py --hybrid [zofesun|namudra|leripel|pubulix]``: prefill and decode throughput of a hybrid decoder beside the decoders of
+"""``bench.py --hybrid [zofesun|namudra|leripel|pubulix|vudivik]``: prefill and decode throughput of a hybrid decoder beside the decoders of
 equal size that the engine already serves (same width, heads, head size, FFN width, layer count, vocabulary; random
 weights, synthetic token ids), all through LLMEngine.generate, and a per-kernel table: each new kernel and the
 like kernel of the closest model as a fraction of the roofline of what bounds it (HBM bytes or matrix / vector
@@ -6,7 +6,9 @@ flops).  Zofesun stands beside Qwen2; Namudra beside Zofesun (the closest: fp32 
 attention kernels) and Qwen2; Leripel beside Namudra (the closest: fp32 residual, retention scan, the same attention
 kernel family, a layer list that is data) and Qwen2; Pubulix beside Leripel (the closest: the same attention kernels
 with a window instead of blocks, experts on the same grouped GEMM, the same convolution and boundary kernels) and
-Qwen2, with Namudra's latent attention as the like kernel of its latent layers."""
+Qwen2, with Namudra's latent attention as the like kernel of its latent layers; Vudivik beside Leripel (the closest: a
+state-space scan behind the same convolution, routed experts on the same grouped GEMM, the same attention kernels) and
+Qwen2, with Pubulix's window attention as the like kernel of its own."""
 from __future__ import annotations
 
 import json
@@ -591,70 +593,202 @@ def _pubulix_kernel_table(dev, H=28, G=4, D=128, W=3584, ff=18944, T=2048, B=64,
     return rows
 
 
-def run_pubulix(args) -> dict:
+def _vudivik_models(name, dev):
+    """Vudivik at a bench size: every layer window attention (1024 positions and the first 16) beside a selective scan
+    (2 W channels of 16 numbers), feed-forwards in turn dense and 16 experts + 2 identity experts (4 per token), the
+    experts' active width equal to the dense one; beside the Leripel and Qwen2 stacks."""
+    from ..models.configs import vudivik_config
+    from ..models.vudivik import VudivikModel
+
+    W, H, G, D, ff, nl, _ = SIZES[name]
+    vc = vudivik_config(f"vudivik-{name}", VOCAB, W, ("dm" * nl)[:nl], heads=H, kv_heads=G, dim=D, ff=ff, window=1024,
+                        keep_first=16, experts=16, identity=2, top=4, expert_ff=(ff // 4) // 64 * 64)
+    mk_l, _, mk_q = _leripel_models(name, dev)
+    return (lambda: VudivikModel(vc, device=dev, seed=1)), mk_l, mk_q
+
+
+def _vudivik_kernel_table(dev, H=28, G=4, D=128, W=3584, ff=18944, T=2048, B=64, ctx=2048, bs=16, win=1024, keep=16, N=16,
+                          E=16, ident=2, top=4):
+    """[(kernel, seconds, bound, fraction of roofline)] for Vudivik's kernels and the like kernels of Leripel (scan,
+    convolution, boundary, router, experts), Pubulix (window attention) and Namudra (normed heads).  The scans are
+    priced in vector issue slots (2 flops each): per state number and token a scalar-decay scan needs 2 (the two
+    multiply-adds), the per-channel one 8 (two products, the exponential at a quarter of the rate, two multiply-adds)."""
+    from ..ops.attention import AttnMetadata, sink_attention
+    from ..ops.elementwise import clamped_glu, qk_norm_store, relu2_, rope_table, rope_vnorm_store
+    from ..ops.moe import moe_experts, moe_route
+    from ..ops.norm import postnorm_residual, residual_rmsnorm
+    from ..ops.recurrent import causal_conv, pad_step_matrix, selective_scan, ssm_scan
+
+    bf = torch.bfloat16
+    i32 = dict(dtype=torch.int32, device=dev)
+    rows = []
+
+    def add(name, sec, flops=0.0, bytes_=0.0, peak=MFMA_BF16):
+        t_c, t_m = flops / peak, bytes_ / HBM_BPS
+        rows.append({"kernel": name, "us": round(sec * 1e6, 1), "bound": "flops" if t_c >= t_m else "bytes",
+                     "roofline_fraction": round(max(t_c, t_m) / sec, 4)})
+
+    nb = T // bs
+    meta = AttnMetadata(q_start=torch.tensor([0, T], **i32), ctx_len=torch.tensor([T], **i32),
+                        block_tables=(torch.arange(nb, **i32) + 1).view(1, nb), slot_mapping=torch.arange(T, **i32) + bs,
+                        max_q_len=T, num_seqs=1, num_tokens=T, state_slots=torch.tensor([0], **i32))
+    nbd = ctx // bs
+    dmeta = AttnMetadata(q_start=torch.arange(B + 1, **i32), ctx_len=torch.full((B,), ctx, **i32),
+                         block_tables=(torch.arange(B * nbd, **i32) + 1).view(B, nbd), slot_mapping=None, max_q_len=1,
+                         num_seqs=B, num_tokens=B, is_decode=True, state_slots=torch.arange(B, **i32))
+    # ---- attention: a window and the first tokens | the window alone
+    kc = torch.randn(nb + 1, G, bs, D, device=dev).to(bf)
+    vc = torch.randn(nb + 1, G, bs, D, device=dev).to(bf)
+    q = torch.randn(T, H, D, device=dev).to(bf)
+    pairs = T * (T + 1) / 2 - (T - win) * (T - win + 1) / 2
+    more = sum(min(keep, max(0, i - win + 1)) for i in range(T))
+    add(f"window attention with kept tokens prefill (window {win} + {keep})",
+        _timed(lambda: sink_attention(q, kc, vc, meta, 0.09, None, window=win, keep=keep)), flops=4.0 * (pairs + more) * H * D)
+    add(f"pubulix window attention prefill (window {win})",
+        _timed(lambda: sink_attention(q, kc, vc, meta, 0.09, None, window=win, softcap=50.0)), flops=4.0 * pairs * H * D)
+    kd = torch.randn(B * nbd + 1, G, bs, D, device=dev).to(bf)
+    vd_ = torch.randn(B * nbd + 1, G, bs, D, device=dev).to(bf)
+    qd = torch.randn(B, H, D, device=dev).to(bf)
+    add(f"window attention with kept tokens decode ({win} + {keep} keys)",
+        _timed(lambda: sink_attention(qd, kd, vd_, dmeta, 0.09, None, window=win, keep=keep)),
+        bytes_=2.0 * B * (win + keep) * G * D * 2)
+    add(f"pubulix window attention decode ({win} keys)",
+        _timed(lambda: sink_attention(qd, kd, vd_, dmeta, 0.09, None, window=win, softcap=50.0)),
+        bytes_=2.0 * B * win * G * D * 2)
+    # ---- biased, normed, rotated heads + K/V store | normed heads + store, rotated heads + store
+    inner, rank = 2 * W, W // 16
+    n = (H + 2 * G) * D
+    proj = torch.randn(T, n + 2 * inner, device=dev).to(bf)
+    pos = torch.arange(T, **i32)
+    tab = rope_table(T, D, 5e5, dev)
+    bias, qw = torch.zeros(n, device=dev), torch.ones(D, device=dev)
+    by = T * n * 2 * 2.0
+    add("rope store with biases and head norms", _timed(lambda: rope_vnorm_store(
+        proj, 0, H * D, (H + G) * D, pos, tab, meta.slot_mapping, kc, vc, H, G, D, D, D, 1e-6, vnorm=False, bias=bias,
+        qw=qw, kw=qw)), bytes_=by)
+    add("leripel rope store", _timed(lambda: rope_vnorm_store(proj, 0, H * D, (H + G) * D, pos, tab, meta.slot_mapping, kc, vc, H, G,
+                                                              D, D, D, 1e-6, vnorm=False)), bytes_=by)
+    add("namudra qk_norm_store (values are the keys)", _timed(lambda: qk_norm_store(
+        proj, 0, H * D, qw, qw, meta.slot_mapping, kc, vc, H, G, D, 1e-6)), bytes_=by)
+    # ---- convolution and scan | leripel's over its own channels and state
+    cw, cb = torch.randn(inner, 4, device=dev) * 0.5, torch.zeros(inner, device=dev)
+    cst = torch.zeros(B + 1, 3, inner, device=dev, dtype=bf)
+    Hs, P, Ns = W // 64, 64, 128
+    ch = Hs * P + 2 * Ns
+    pj = (torch.randn(T, 2 * Hs * P + 2 * Ns + Hs, device=dev) * 0.5).to(bf)
+    cws, cbs = torch.randn(ch, 4, device=dev) * 0.5, torch.zeros(ch, device=dev)
+    csts = torch.zeros(B + 1, 3, ch, device=dev, dtype=bf)
+    add("causal_conv prefill (4 taps)", _timed(lambda: causal_conv(proj, n, cw, cb, cst, meta)), bytes_=T * inner * 2 * 2.0)
+    add("leripel causal_conv prefill (4 taps)", _timed(lambda: causal_conv(pj, Hs * P, cws, cbs, csts, meta)), bytes_=T * ch * 2 * 2.0)
+    projd = proj[:B].contiguous()
+    pjd = pj[:B].contiguous()
+    add("causal_conv decode", _timed(lambda: causal_conv(projd, n, cw, cb, cst, dmeta)), bytes_=B * inner * 2 * (2 + 2 * 3.0))
+    add("leripel causal_conv decode", _timed(lambda: causal_conv(pjd, Hs * P, cws, cbs, csts, dmeta)), bytes_=B * ch * 2 * (2 + 2 * 3.0))
+    xc = causal_conv(proj, n, cw, cb, cst, meta)
+    low = torch.randn(T, rank + 2 * N, device=dev).to(bf)
+    wdt = pad_step_matrix(torch.randn(inner, rank, device=dev) * rank ** -0.5).to(bf).contiguous()
+    dtb, dsk = torch.full((inner,), -3.0, device=dev), torch.ones(inner, device=dev)
+    A = -torch.rand(inner, N, device=dev) * N - 0.1
+    sst = torch.zeros(B + 1, inner, N, device=dev)
+    ssp = torch.zeros(B + 1, Hs, Ns, P, device=dev)
+    z1, a1, d1 = torch.zeros(Hs, device=dev), torch.zeros(Hs, device=dev), torch.ones(Hs, device=dev)
+    add(f"selective_scan prefill (1 x {T}, step sizes and gate inside)",
+        _timed(lambda: selective_scan(xc, low, wdt, rank, dtb, A, dsk, proj, n + inner, sst, meta), 5, 1),
+        flops=16.0 * T * inner * N, bytes_=T * inner * 2 * 3.0, peak=VALU_F32)
+    xbc = causal_conv(pj, Hs * P, cws, cbs, csts, meta)
+    add(f"leripel ssm_scan prefill (1 x {T})", _timed(lambda: ssm_scan(xbc, pj, Hs * P + ch, z1, a1, d1, ssp, meta, Hs, 1, Ns, P), 5, 1),
+        flops=4.0 * T * Hs * Ns * P, bytes_=T * ch * 2.0, peak=VALU_F32)
+    q4 = torch.arange(5, **i32) * (T // 4)
+    m4 = AttnMetadata(q_start=q4, ctx_len=torch.full((4,), T // 4, **i32), block_tables=meta.block_tables.expand(4, -1),
+                      slot_mapping=meta.slot_mapping, max_q_len=T // 4, num_seqs=4, num_tokens=T, state_slots=torch.arange(4, **i32))
+    add(f"selective_scan prefill (4 x {T // 4})",
+        _timed(lambda: selective_scan(xc, low, wdt, rank, dtb, A, dsk, proj, n + inner, sst, m4), 5, 1),
+        flops=16.0 * T * inner * N, bytes_=T * inner * 2 * 3.0, peak=VALU_F32)
+    add(f"leripel ssm_scan prefill (4 x {T // 4})", _timed(lambda: ssm_scan(xbc, pj, Hs * P + ch, z1, a1, d1, ssp, m4, Hs, 1, Ns, P), 5, 1),
+        flops=4.0 * T * Hs * Ns * P, bytes_=T * ch * 2.0, peak=VALU_F32)
+    xcd, lowd = xc[:B].contiguous(), low[:B].contiguous()
+    add("selective_scan decode (step sizes and gate inside)",
+        _timed(lambda: selective_scan(xcd, lowd, wdt, rank, dtb, A, dsk, projd, n + inner, sst, dmeta)),
+        bytes_=2.0 * B * inner * N * 4 + 2.0 * inner * rank)
+    xbd = xbc[:B].contiguous()
+    add("leripel ssm_scan decode", _timed(lambda: ssm_scan(xbd, pjd, Hs * P + ch, z1, a1, d1, ssp, dmeta, Hs, 1, Ns, P)),
+        bytes_=2.0 * B * Hs * Ns * P * 4)
+    # ---- boundary: normed outputs | leripel's sums of the same operands
+    x = torch.randn(T, W, device=dev)
+    a, b = torch.randn(T, W, device=dev).to(bf), torch.randn(T, W, device=dev).to(bf)
+    e = torch.randn(T, top, W, device=dev).to(bf)
+    ec, idw, w32 = torch.rand(T, top, device=dev), torch.rand(T, device=dev), torch.ones(W, device=dev)
+    add("postnorm_residual (two mixers)", _timed(lambda: postnorm_residual(x, a, w32, b, w32, 0.5, w=w32, mult=0.7)),
+        bytes_=T * W * (8 + 2.0 * 2 + 2))
+    add("leripel residual_rmsnorm (two branches)", _timed(lambda: residual_rmsnorm(x, a, b, w=w32)), bytes_=T * W * (8 + 2.0 * 2 + 2))
+    add(f"postnorm_residual (sum of {top} experts + identity)",
+        _timed(lambda: postnorm_residual(x, e=e, ecoef=ec, idw=idw, w=w32, mult=0.7)), bytes_=T * W * (8 + 2.0 * top + 2))
+    add(f"leripel residual_rmsnorm (sum of {top} experts)", _timed(lambda: residual_rmsnorm(x, e=e, ecoef=ec, w=w32)),
+        bytes_=T * W * (8 + 2.0 * top + 2))
+    xd, ad, bd = x[:B].contiguous(), a[:B].contiguous(), b[:B].contiguous()
+    add("postnorm_residual (two mixers), decode rows", _timed(lambda: postnorm_residual(xd, ad, w32, bd, w32, 0.5, w=w32, mult=0.7)),
+        bytes_=B * W * (8 + 2.0 * 2 + 2))
+    add("leripel residual_rmsnorm (two branches), decode rows", _timed(lambda: residual_rmsnorm(xd, ad, bd, w=w32)),
+        bytes_=B * W * (8 + 2.0 * 2 + 2))
+    # ---- feed-forward: router, experts, squared relu | leripel's router and SiLU experts, the clamped GLU
+    F = (ff // 4) // 64 * 64
+    wr = torch.randn(E + ident, W, device=dev) * 0.05
+    corr = torch.zeros(E + ident, device=dev)
+    add(f"moe_route ({E} + {ident} rows, correction, fp32 input)",
+        _timed(lambda: moe_route(x, wr, E + ident, top, corr=corr, identity=ident)), flops=2.0 * T * (E + ident) * W,
+        bytes_=T * W * 4.0, peak=VALU_F32)
+    add(f"leripel moe_route ({E} rows, groups)", _timed(lambda: moe_route(a, wr[:E].contiguous(), E, top, 4, 2)), flops=2.0 * T * E * W,
+        bytes_=T * W * 2.0, peak=VALU_F32)
+    ids, _, _ = moe_route(a, wr[:E].contiguous(), E, top)  # (every choice a real expert: the whole product is timed)
+    wgu = (torch.randn(E, 2 * F, W, device=dev) * 0.02).to(bf)
+    wu = wgu[:, :F].contiguous()
+    wd = (torch.randn(E, W, F, device=dev) * 0.02).to(bf)
+    add(f"squared-relu experts prefill ({T} x {top} rows)", _timed(lambda: moe_experts(a, ids, wu, wd, unit="relu2")),
+        flops=4.0 * T * top * F * W)
+    add(f"leripel SiLU experts prefill ({T} x {top} rows)", _timed(lambda: moe_experts(a, ids, wgu, wd)), flops=6.0 * T * top * F * W)
+    idd = ids[:B].contiguous()
+    add(f"squared-relu experts decode ({B} x {top} rows)", _timed(lambda: moe_experts(ad, idd, wu, wd, unit="relu2")),
+        bytes_=2.0 * E * F * W * 2)
+    add(f"leripel SiLU experts decode ({B} x {top} rows)", _timed(lambda: moe_experts(ad, idd, wgu, wd)), bytes_=3.0 * E * F * W * 2)
+    u = torch.randn(T, ff, device=dev).to(bf)
+    gu = torch.randn(T, 2 * ff, device=dev).to(bf)
+    add("squared relu (in place)", _timed(lambda: relu2_(u)), bytes_=T * ff * 2 * 2.0)
+    add("leripel SiLU-gated unit", _timed(lambda: clamped_glu(gu, None, 1.0, 0.0)), bytes_=T * ff * 2 * 3.0)
+    return rows
+
+
+def _run_family(names, models, kernel_table) -> dict:
+    """A hybrid decoder beside the decoders of equal size: ``names`` (the new one first), ``models`` (size, device) ->
+    their constructors in the same order."""
     dev = torch.device("cuda", 0)
     torch.cuda.set_device(dev)
     sizes = {}
     for name in SIZES:
-        makers = dict(zip(("pubulix", "leripel", "qwen2"), _pubulix_models(name, dev)))
+        makers = dict(zip(names, models(name, dev)))
         cell = {}
         for batch, plen, glen in ((8, 2048, 64), (64, 1024, 64)):
             key = f"B{batch}_P{plen}_G{glen}"
             cell[key] = {k: _engine_numbers(mk, dev, batch, plen, glen) for k, mk in makers.items()}
             print(json.dumps({"size": name, "shape": key, **cell[key]}), flush=True)
         sizes[name] = cell
-    kernels = _pubulix_kernel_table(dev)
+    kernels = kernel_table(dev)
     for r in kernels:
         print(json.dumps(r), flush=True)
-    return {"metric": "pubulix_vs_leripel_vs_qwen2_tokens_per_s", "unit": "tokens/s", "dtype": "bf16",
-            "data": "synthetic", "sizes": sizes, "kernels": kernels}
+    return {"metric": "_vs_".join(names) + "_tokens_per_s", "unit": "tokens/s", "dtype": "bf16", "data": "synthetic",
+            "sizes": sizes, "kernels": kernels}
 
 
-def run_leripel(args) -> dict:
-    dev = torch.device("cuda", 0)
-    torch.cuda.set_device(dev)
-    sizes = {}
-    for name in SIZES:
-        makers = dict(zip(("leripel", "namudra", "qwen2"), _leripel_models(name, dev)))
-        cell = {}
-        for batch, plen, glen in ((8, 2048, 64), (64, 1024, 64)):
-            key = f"B{batch}_P{plen}_G{glen}"
-            cell[key] = {k: _engine_numbers(mk, dev, batch, plen, glen) for k, mk in makers.items()}
-            print(json.dumps({"size": name, "shape": key, **cell[key]}), flush=True)
-        sizes[name] = cell
-    kernels = _leripel_kernel_table(dev)
-    for r in kernels:
-        print(json.dumps(r), flush=True)
-    return {"metric": "leripel_vs_namudra_vs_qwen2_tokens_per_s", "unit": "tokens/s", "dtype": "bf16",
-            "data": "synthetic", "sizes": sizes, "kernels": kernels}
-
-
-def run_namudra(args) -> dict:
-    dev = torch.device("cuda", 0)
-    torch.cuda.set_device(dev)
-    sizes = {}
-    for name in SIZES:
-        makers = dict(zip(("namudra", "zofesun", "qwen2"), _namudra_models(name, dev)))
-        cell = {}
-        for batch, plen, glen in ((8, 2048, 64), (64, 1024, 64)):
-            key = f"B{batch}_P{plen}_G{glen}"
-            cell[key] = {k: _engine_numbers(mk, dev, batch, plen, glen) for k, mk in makers.items()}
-            print(json.dumps({"size": name, "shape": key, **cell[key]}), flush=True)
-        sizes[name] = cell
-    kernels = _namudra_kernel_table(dev)
-    for r in kernels:
-        print(json.dumps(r), flush=True)
-    return {"metric": "namudra_vs_zofesun_vs_qwen2_tokens_per_s", "unit": "tokens/s", "dtype": "bf16",
-            "data": "synthetic", "sizes": sizes, "kernels": kernels}
+FAMILIES = {
+    "namudra": (("namudra", "zofesun", "qwen2"), _namudra_models, _namudra_kernel_table),
+    "leripel": (("leripel", "namudra", "qwen2"), _leripel_models, _leripel_kernel_table),
+    "pubulix": (("pubulix", "leripel", "qwen2"), _pubulix_models, _pubulix_kernel_table),
+    "vudivik": (("vudivik", "leripel", "qwen2"), _vudivik_models, _vudivik_kernel_table),
+}
 
 
 def run(args) -> dict:
-    if getattr(args, "hybrid", None) == "namudra":
-        return run_namudra(args)
-    if getattr(args, "hybrid", None) == "leripel":
-        return run_leripel(args)
-    if getattr(args, "hybrid", None) == "pubulix":
-        return run_pubulix(args)
+    if getattr(args, "hybrid", None) in FAMILIES:
+        return _run_family(*FAMILIES[args.hybrid])
     dev = torch.device("cuda", 0)
     torch.cuda.set_device(dev)
     sizes = {}
