@@ -101,6 +101,67 @@ __device__ void route_select(float* z, int E, int R, int top, int ngroups, int k
   if (rx.idw != nullptr) rx.idw[t] = idsum;
 }
 
+// The same by a whole wave (one group of experts): lane l holds the rows l, l + 64, ... of the logits z, every choice is a
+// wave-wide maximum (ties to the lower index).  All 64 lanes call it with the same arguments.
+__device__ void route_select_wave(const float* z, int E, int R, int top, int t, int* __restrict__ ids,
+                                  float* __restrict__ wts, float* __restrict__ sgate, const RouteExtra& rx) {
+  const int lane = threadIdx.x & 63;
+  constexpr int PER = RT_MAXR / 64;
+  if (lane == 0 && R > E && sgate != nullptr) sgate[t] = 1.f / (1.f + expf(-z[E]));
+  float zl[PER], mx = -INFINITY, sum = 0.f;
+#pragma unroll
+  for (int j = 0; j < PER; ++j) {
+    zl[j] = lane + 64 * j < E ? z[lane + 64 * j] : -INFINITY;
+    mx = fmaxf(mx, zl[j]);
+  }
+  mx = wave_max(mx);
+#pragma unroll
+  for (int j = 0; j < PER; ++j) {
+    zl[j] = expf(zl[j] - mx);  // (rows past E: 0)
+    sum += zl[j];
+  }
+  const float inv = 1.f / wave_sum(sum);
+  float pick[PER];  // what the choice goes by; -inf: taken, or no row
+#pragma unroll
+  for (int j = 0; j < PER; ++j) {
+    zl[j] *= inv;
+    const int e = lane + 64 * j;
+    pick[j] = e < E ? zl[j] + (rx.corr ? rx.corr[e] : 0.f) : -INFINITY;
+  }
+  float idsum = 0.f;
+  for (int n = 0; n < top; ++n) {
+    float bv = -INFINITY, bw = 0.f;
+    int be = RT_MAXR;
+#pragma unroll
+    for (int j = 0; j < PER; ++j)
+      if (pick[j] > bv) {
+        bv = pick[j];
+        bw = zl[j];
+        be = lane + 64 * j;
+      }
+#pragma unroll
+    for (int o = 32; o > 0; o >>= 1) {
+      const float ov = __shfl_xor(bv, o, 64), ow = __shfl_xor(bw, o, 64);
+      const int oe = __shfl_xor(be, o, 64);
+      if (ov > bv || (ov == bv && oe < be)) {
+        bv = ov;
+        bw = ow;
+        be = oe;
+      }
+    }
+#pragma unroll
+    for (int j = 0; j < PER; ++j)
+      if (be == lane + 64 * j) pick[j] = -INFINITY;
+    const bool none = be >= E, ident = !none && be >= E - rx.nid;
+    if (ident) idsum += bw;
+    if (lane == 0) {
+      ids[(size_t)t * top + n] = none ? 0 : be;
+      wts[(size_t)t * top + n] = none || ident ? 0.f : bw;
+    }
+  }
+  if (lane == 0 && rx.idw != nullptr) rx.idw[t] = idsum;
+}
+
 // h [T][ld] (the normed layer input); wr [R][W] fp32, rows 0 .. E-1 the experts, row E (R = E + 1) the shared expert's
 // gate.  ids [T][top] int32, wts [T][top] fp32 (the chosen experts by falling score; ties to the lower index),
 // sgate [T] fp32 = sigmoid(row E's logit).  grid (ceil(T / RT_TOK)), 256 threads: thread (token tid % 16, part
@@ -194,6 +255,11 @@ moe_route_kernel(const T* __restrict__ h, int ld, const float* __restrict__ wr, 
   for (int j = 0; j < RT_MAXR / 16; ++j)
     if (part + 16 * j < R) lgs[tok * (R + 1) + part + 16 * j] = acc[j];
   __syncthreads();
+  if (ngroups == 1) {
+    for (int i = threadIdx.x >> 6; i < RT_TOK && t0 + i < T_; i += 4)
+      route_select_wave(lgs + i * (R + 1), E, R, top, t0 + i, ids, wts, sgate, rx);
+    return;
+  }
   if (threadIdx.x >= RT_TOK || t0 + threadIdx.x >= T_) return;
   route_select(lgs + threadIdx.x * (R + 1), E, R, top, ngroups, keep, t0 + threadIdx.x, ids, wts, sgate, rx);
 }
@@ -240,6 +306,10 @@ moe_route_rows_kernel(const T* __restrict__ h, int ld, const float* __restrict__
     if (lane == 0) z[r] = a;
   }
   __syncthreads();
+  if (ngroups == 1) {
+    if (wid == 0) route_select_wave(z, E, R, top, t, ids, wts, sgate, rx);
+    return;
+  }
   if (threadIdx.x == 0) route_select(z, E, R, top, ngroups, keep, t, ids, wts, sgate, rx);
 }
 

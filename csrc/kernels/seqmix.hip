@@ -180,6 +180,94 @@ __global__ void rope_vnorm_store_kernel(const T* __restrict__ proj, int ld, int 
   }
 }
 
+// The same in 16-byte accesses (bf16; d, vd and rd multiples of 16, d <= 256, halves rotated, values without RMS division):
+// a lane owns 16 elements of a head -- 8 of the first rotated half and the 8 they are paired with, or 16 consecutive ones
+// past the rotated part -- and LG lanes a head, so a head's sum of squares stays inside LG lanes.
+// grid (ceil(T (H + 2 G) LG / 256)), 256 threads: (token, head) pairs in a row, q heads, then k heads, then v heads.
+template <int LG>
+__global__ void __launch_bounds__(256)
+rope_store_vec_kernel(const bf16* __restrict__ proj, int ld, int qoff, int koff, int voff, const int* __restrict__ positions,
+                      const float* __restrict__ table, int table_rows, const int* __restrict__ slot_mapping,
+                      bf16* __restrict__ q_out, bf16* __restrict__ k_cache, bf16* __restrict__ v_cache, int T_, int H, int G,
+                      int d, int vd, int rd, int BS, long nslots, float eps, const float* __restrict__ bias,
+                      const float* __restrict__ qw, const float* __restrict__ kw) {
+  const int nh = H + 2 * G;
+  const long pair = ((long)blockIdx.x * 256 + threadIdx.x) / LG;
+  const int u = threadIdx.x % LG;
+  const bool live = pair < (long)T_ * nh;
+  const int t = live ? (int)(pair / nh) : 0, hb = live ? (int)(pair - (long)t * nh) : 0;
+  const bool isq = hb < H, isv = hb >= H + G;
+  const int hh = isq ? hb : isv ? hb - H - G : hb - H;
+  const int n = isv ? vd : d, off = (isq ? qoff : isv ? voff : koff) + hh * n;
+  const int half = rd >> 1;
+  const bool rot = !isv && 8 * u < half;
+  // the lane's two runs of 8: first elements i0 and i1 (n: none)
+  const int i0 = rot ? 8 * u : 16 * u, i1 = rot ? 8 * u + half : i0 + 8;
+  const bool on = live && i0 < n;
+  float a[8], b[8];
+  bf16x8_t va = bf16x8_t{0, 0, 0, 0, 0, 0, 0, 0}, vb = va;
+  const bf16* row = proj + (size_t)t * ld + off;
+  if (on) {
+    va = *reinterpret_cast<const bf16x8_t*>(row + i0);
+    vb = *reinterpret_cast<const bf16x8_t*>(row + i1);
+  }
+  unpack8(va, a);
+  unpack8(vb, b);
+  auto add8 = [](float* v, const float* p) {
+    const f32x4_t x = *reinterpret_cast<const f32x4_t*>(p), y = *reinterpret_cast<const f32x4_t*>(p + 4);
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+      v[e] += x[e];
+      v[4 + e] += y[e];
+    }
+  };
+  if (bias && on) {
+    add8(a, bias + off + i0);
+    add8(b, bias + off + i1);
+  }
+  const float* nw = isv ? nullptr : isq ? qw : kw;
+  float ss = 0.f;
+#pragma unroll
+  for (int e = 0; e < 8; ++e) ss = fmaf(a[e], a[e], fmaf(b[e], b[e], ss));
+#pragma unroll
+  for (int o = LG / 2; o > 0; o >>= 1) ss += __shfl_xor(ss, o, 64);
+  if (!on) return;
+  if (nw) {
+    const float r = 1.f / sqrtf(ss / (float)n + eps);
+#pragma unroll
+    for (int e = 0; e < 8; ++e) {
+      a[e] *= r * nw[i0 + e];
+      b[e] *= r * nw[i1 + e];
+    }
+  }
+  if (rot) {
+    const int pos = positions[t];
+    if (index_ok(pos, table_rows, ERR_ROPE_POS)) {
+      const float* cs = table + (size_t)pos * rd + i0;
+      float c[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f}, s[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
+      add8(c, cs);
+      add8(s, cs + half);
+#pragma unroll
+      for (int e = 0; e < 8; ++e) {
+        const float x = a[e], y = b[e];
+        a[e] = x * c[e] - y * s[e];
+        b[e] = y * c[e] + x * s[e];
+      }
+    }
+  }
+  bf16* dst;
+  if (isq) {
+    dst = q_out + ((size_t)t * H + hh) * d;
+  } else {
+    const int slot = slot_mapping[t];
+    if (slot < 0 || !index_ok(slot, nslots, ERR_KV_SLOT)) return;
+    const int blk = slot / BS, o = slot % BS;
+    dst = (isv ? v_cache : k_cache) + (((size_t)blk * G + hh) * BS + o) * n;
+  }
+  *reinterpret_cast<bf16x8_t*>(dst + i0) = pack8(a);
+  *reinterpret_cast<bf16x8_t*>(dst + i1) = pack8(b);
+}
+
 // ------------------------------------------------------------------------------------------------ sink attention
 // softmax over the visible keys plus one key-less, value-less term exp(sink_h) in the denominator: the running
 // (max, sum) starts at (sink_h, 1) instead of (-inf, 0).
@@ -1356,6 +1444,26 @@ GRAG_API hipError_t grag_rope_vnorm_store(const void* proj, int ld, int qoff, in
                                           const float* qw, const float* kw, hipStream_t st) {
   if (T_ <= 0) return hipSuccess;
   if (H + 2 * G > 4 * 65535) return hipErrorInvalidValue;
+  auto al16 = [](const void* p) { return (reinterpret_cast<uintptr_t>(p) & 15) == 0; };
+  if (dt == 0 && flags == 2 && d % 16 == 0 && vd % 16 == 0 && rd % 16 == 0 && d <= 256 && vd <= 256 && ld % 8 == 0 &&
+      qoff % 8 == 0 && koff % 8 == 0 && voff % 8 == 0 && al16(proj) && al16(q_out) && al16(k_cache) && al16(v_cache) &&
+      al16(table) && al16(bias)) {
+    const int units = (d > vd ? d : vd) / 16;
+    const int LG = units <= 1 ? 1 : units <= 2 ? 2 : units <= 4 ? 4 : units <= 8 ? 8 : 16;
+    const long lanes = (long)T_ * (H + 2 * G) * LG;
+    const dim3 vgrid((unsigned)((lanes + 255) / 256));
+#define ROPE_VEC(L)                                                                                                       \
+  hipLaunchKernelGGL(rope_store_vec_kernel<L>, vgrid, dim3(256), 0, st, (const bf16*)proj, ld, qoff, koff, voff,          \
+                     positions, table, table_rows, slot_mapping, (bf16*)q_out, (bf16*)k_cache, (bf16*)v_cache, T_, H, G,  \
+                     d, vd, rd, BS, nslots, eps, bias, qw, kw)
+    if (LG == 1) ROPE_VEC(1);
+    else if (LG == 2) ROPE_VEC(2);
+    else if (LG == 4) ROPE_VEC(4);
+    else if (LG == 8) ROPE_VEC(8);
+    else ROPE_VEC(16);
+#undef ROPE_VEC
+    return hipGetLastError();
+  }
   DT_DISPATCH(dt, hipLaunchKernelGGL(rope_vnorm_store_kernel<T>, dim3(T_, (H + 2 * G + 3) / 4), dim3(256), 0, st, (const T*)proj, ld, qoff,
                                      koff, voff, positions, table, table_rows, slot_mapping, (T*)q_out, (T*)k_cache,
                                      (T*)v_cache, H, G, d, vd, rd, BS, nslots, eps, flags, bias, qw, kw);)

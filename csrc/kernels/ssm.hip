@@ -25,6 +25,35 @@ template <> __device__ __forceinline__ void sts<float>(float* p, float v) { *p =
 __device__ __forceinline__ float silu_f(float x) { return x / (1.f + expf(-x)); }
 __device__ __forceinline__ float softplus_f(float x) { return x > 20.f ? x : log1pf(expf(x)); }
 
+// softplus out of the hardware's log2 / exp2: log(1 + u), u = e^-|x|, by its series for small u (where 1 + u would round
+// u away), else through w = 1 + u with the rounding of w divided out: log(w) u / (w - 1)
+__device__ __forceinline__ float softplus_hw(float x) {
+  constexpr float LOG2E = 1.4426950408889634f, LN2 = 0.6931471805599453f;
+  const float u = __builtin_amdgcn_exp2f(-fabsf(x) * LOG2E);
+  const float series = u * fmaf(u, fmaf(u, fmaf(u, fmaf(u, 0.2f, -0.25f), 0.33333334f), -0.5f), 1.f);
+  const float w = 1.f + u;
+  const float lg = LN2 * __builtin_amdgcn_logf(w) * u * __builtin_amdgcn_rcpf(w - 1.f);
+  return fmaxf(x, 0.f) + (u < 0.0625f ? series : lg);
+}
+// SiLU of a value that is stored as bf16 (hardware exp2 and reciprocal) or as fp32
+template <typename T> __device__ __forceinline__ float silu_t(float x) {
+  if (sizeof(T) == 2) return x * __builtin_amdgcn_rcpf(1.f + __builtin_amdgcn_exp2f(-1.4426950408889634f * x));
+  return silu_f(x);
+}
+
+// 4 consecutive elements
+template <typename T> __device__ __forceinline__ f32x4_t ld4s(const T* p);
+template <> __device__ __forceinline__ f32x4_t ld4s<float>(const float* p) { return *reinterpret_cast<const f32x4_t*>(p); }
+template <> __device__ __forceinline__ f32x4_t ld4s<bf16>(const bf16* p) {
+  const bf16x4_t v = *reinterpret_cast<const bf16x4_t*>(p);
+  return f32x4_t{bits2f(v[0]), bits2f(v[1]), bits2f(v[2]), bits2f(v[3])};
+}
+template <typename T> __device__ __forceinline__ void st4s(T* p, f32x4_t v);
+template <> __device__ __forceinline__ void st4s<float>(float* p, f32x4_t v) { *reinterpret_cast<f32x4_t*>(p) = v; }
+template <> __device__ __forceinline__ void st4s<bf16>(bf16* p, f32x4_t v) {
+  *reinterpret_cast<bf16x4_t*>(p) = bf16x4_t{f2bits(v[0]), f2bits(v[1]), f2bits(v[2]), f2bits(v[3])};
+}
+
 // ------------------------------------------------------------------------------------------------ causal convolution
 constexpr int CONV_MAX_TAPS = 16;
 constexpr int CONV_TT = 16;  // tokens per workgroup
@@ -83,6 +112,79 @@ causal_conv_kernel(const T* __restrict__ proj, int ld, int coff, int C, int taps
 #pragma unroll
     for (int j = 0; j < CONV_MAX_TAPS - 1; ++j)
       if (j < taps - 1) sts(dst + (size_t)j * C + c, win[j]);
+  }
+}
+
+// The same for up to MT taps and rows in groups of four channels (C, ld, coff multiples of 4, aligned pointers): a thread
+// owns four channels of a token tile, all of whose inputs are in flight before the first sum.  The weights stand at the
+// end of MT places (zeros before them), so every register index is known when the kernel is compiled.
+// grid (ceil(C / 1024), ceil(max_q_len / CONV_TT), nseq); the mode bits as above.
+template <typename T, int MT>
+__global__ void __launch_bounds__(256)
+causal_conv_vec_kernel(const T* __restrict__ proj, int ld, int coff, int C, int taps, const float* __restrict__ w,
+                       const float* __restrict__ b, T* __restrict__ cstate, const int* __restrict__ slots,
+                       const int* __restrict__ q_start, const int* __restrict__ ctx_len, T* __restrict__ out, int nslots,
+                       int mode) {
+  const int seq = blockIdx.z, c = (blockIdx.x * 256 + threadIdx.x) * 4;
+  const int qa = q_start[seq], qlen = q_start[seq + 1] - qa;
+  const int t0 = blockIdx.y * CONV_TT;
+  if (t0 >= qlen || c >= C) return;
+  const bool fresh = ctx_len[seq] - qlen == 0;
+  const int slot = slots[seq];
+  const bool slot_ok = fresh || index_ok(slot, nslots, ERR_SAMPLER_SLOT);
+  const T* st = cstate + (size_t)(slot_ok && !fresh ? slot : 0) * (taps - 1) * C + c;
+  const T* in = proj + (size_t)qa * ld + coff + c;
+  const int nt = min(CONV_TT, qlen - t0), lead = MT - taps;
+  f32x4_t x[MT - 1 + CONV_TT];  // x[MT - 1 + tt] = input of token t0 + tt
+#pragma unroll
+  for (int tt = 0; tt < CONV_TT; ++tt)
+    x[MT - 1 + tt] = tt < nt ? ld4s(in + (size_t)(t0 + tt) * ld) : f32x4_t{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+  for (int j = 0; j < MT - 1; ++j) {
+    x[j] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+    const int s = t0 - (MT - 1) + j;  // token index in the portion
+    if (j >= lead) {
+      if (s >= 0) x[j] = ld4s(in + (size_t)s * ld);
+      else if (!fresh && slot_ok) x[j] = ld4s(st + (size_t)(taps - 1 + s) * C);
+    }
+  }
+  float wt[MT][4];
+#pragma unroll
+  for (int j = 0; j < MT; ++j)
+#pragma unroll
+    for (int v = 0; v < 4; ++v) wt[j][v] = j >= lead ? w[(size_t)(c + v) * taps + j - lead] : 0.f;
+  const f32x4_t bias = b ? *reinterpret_cast<const f32x4_t*>(b + c) : f32x4_t{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+  for (int tt = 0; tt < CONV_TT; ++tt) {
+    if (tt >= nt) break;
+    f32x4_t acc = bias;
+#pragma unroll
+    for (int j = 0; j < MT; ++j)
+#pragma unroll
+      for (int v = 0; v < 4; ++v) acc[v] = fmaf(wt[j][v], x[tt + j][v], acc[v]);
+    if (!(mode & 1)) {
+#pragma unroll
+      for (int v = 0; v < 4; ++v) acc[v] = silu_t<T>(acc[v]);
+    }
+    if (mode & 2) acc += x[MT - 1 + tt];
+    st4s(out + (size_t)(qa + t0 + tt) * C + c, acc);
+  }
+  if ((mode & 4) && taps > 1 && index_ok(slot, nslots, ERR_SAMPLER_SLOT)) {  // (t0 is 0: one tile holds the portion)
+    T* dst = cstate + (size_t)slot * (taps - 1) * C + c;
+#pragma unroll
+    for (int j = 0; j < MT - 1; ++j) {
+      if (j < lead) continue;
+      const int s = nt - (MT - 1) + j;  // the token whose input stands at place j after the step
+      f32x4_t v = f32x4_t{0.f, 0.f, 0.f, 0.f};
+      if (s >= 0) {
+        v = ld4s(in + (size_t)s * ld);
+      } else {
+#pragma unroll
+        for (int k = 0; k < MT - 1; ++k)
+          if (k == nt + j) v = x[k];
+      }
+      st4s(dst + (size_t)(j - lead) * C, v);
+    }
   }
 }
 
@@ -382,7 +484,7 @@ chan_scan_kernel(const T* __restrict__ xc, const T* __restrict__ low, int low_ld
     __syncthreads();  // the tile before is consumed
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
-      const float dt = softplus_f(dv[i]);
+      const float dt = softplus_hw(dv[i]);
       sd[4 * quad + i][16 * wid + ql] = f32x2_t{dt * LOG2E, dt * xv[i]};
     }
     for (int idx = threadIdx.x; idx < nb * 2 * NP; idx += 256) {
@@ -390,6 +492,7 @@ chan_scan_kernel(const T* __restrict__ xc, const T* __restrict__ low, int low_ld
       bc[t][r / NP][n] = n < N ? lds(low + (size_t)(qa + t0 + t) * low_ld + R + (r < NP ? 0 : N) + n) : 0.f;
     }
     __syncthreads();
+#pragma unroll 4
     for (int t = 0; t < nb; ++t) {
       const f32x2_t d = sd[t][cl];
       float y = 0.f;
@@ -415,7 +518,7 @@ chan_scan_kernel(const T* __restrict__ xc, const T* __restrict__ low, int low_ld
         const int t = 4 * quad + i;
         if (t < nb && sc_ok) {
           const float zv = lds(proj + (size_t)(qa + t0 + t) * ld + zoff + sc);
-          sts(out + (size_t)(qa + t0 + t) * inner + sc, fmaf(dsk, xv[i], sy[t][16 * wid + ql]) * silu_f(zv));
+          sts(out + (size_t)(qa + t0 + t) * inner + sc, fmaf(dsk, xv[i], sy[t][16 * wid + ql]) * silu_t<T>(zv));
         }
       }
     }
@@ -436,6 +539,168 @@ chan_scan_kernel(const T* __restrict__ xc, const T* __restrict__ low, int low_ld
     }
   }
   if (MODE == 1 && part == 0 && ch_ok) wa[(size_t)(seq * maxchunks + chunk) * inner + ch] = dtsum;
+}
+
+// One token per sequence (decode rows): the same with sequences in the place of tokens.  grid (ceil(inner / 64),
+// ceil(nseq / SB)): a workgroup takes 64 channels of SB <= SC_TB sequences, so the step-size matrix is read once for all of
+// them.  States travel G sequences at a time, the next group's loads in flight during the sums of the one before.
+template <typename T, int NPT, int G>
+__global__ void __launch_bounds__(256)
+chan_step_kernel(const T* __restrict__ xc, const T* __restrict__ low, int low_ld, const T* __restrict__ wdt, int R, int Rp,
+                 const float* __restrict__ dt_bias, const float* __restrict__ A, const float* __restrict__ Dv,
+                 const T* __restrict__ proj, int ld, int zoff, float* __restrict__ state, const int* __restrict__ slots,
+                 const int* __restrict__ q_start, const int* __restrict__ ctx_len, T* __restrict__ out, int nseq, int SB,
+                 int inner, int N, int nslots) {
+  constexpr float LOG2E = 1.4426950408889634f;
+  constexpr int NP = 4 * NPT;
+  typedef float f32x2_t __attribute__((ext_vector_type(2)));
+  __shared__ __attribute__((aligned(16))) float bc[SC_TB][2][NP];
+  __shared__ __attribute__((aligned(16))) f32x2_t sd[SC_TB][SC_CH];
+  __shared__ float sy[SC_TB][SC_CH];
+  __shared__ int srow[SC_TB], sslot[SC_TB], sfresh[SC_TB];  // token row (-1: no token), slot (-1: none), starts from zeros
+  const int s0 = blockIdx.y * SB, ns = min(SB, nseq - s0), c0 = blockIdx.x * SC_CH;
+  if (threadIdx.x < SC_TB) {
+    int row = -1, slot = -1, fresh = 1;
+    if (threadIdx.x < ns) {
+      const int s = s0 + threadIdx.x, qa = q_start[s];
+      if (q_start[s + 1] > qa) {
+        row = qa;
+        fresh = ctx_len[s] == 1;
+        slot = slots[s];
+        if (!index_ok(slot, nslots, ERR_SAMPLER_SLOT)) slot = -1;
+      }
+    }
+    srow[threadIdx.x] = row;
+    sslot[threadIdx.x] = slot;
+    sfresh[threadIdx.x] = fresh;
+  }
+  const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6, ql = lane & 15, quad = lane >> 4;
+  const int cl = threadIdx.x >> 2, part = threadIdx.x & 3, ch = c0 + cl;
+  const bool ch_ok = ch < inner, vecn = (N & 3) == 0;
+  float a2[NPT];
+#pragma unroll
+  for (int j = 0; j < NPT; ++j) {
+    const int n = 4 * (part + 4 * (j >> 2)) + (j & 3);
+    a2[j] = ch_ok && n < N ? A[(size_t)ch * N + n] : 0.f;
+  }
+  __syncthreads();
+  auto load = [&](int i, float (&S)[NPT]) {
+    const bool use = i < ns && ch_ok && sslot[i < SC_TB ? i : 0] >= 0 && !sfresh[i < SC_TB ? i : 0];
+    const float* sp = state + ((size_t)(use ? sslot[i] : 0) * inner + (use ? ch : 0)) * N;
+#pragma unroll
+    for (int j = 0; j < NPT / 4; ++j) {
+      const int n0 = 4 * (part + 4 * j);
+      f32x4_t v = f32x4_t{0.f, 0.f, 0.f, 0.f};
+      if (use && n0 < N) {
+        if (vecn) {
+          v = *reinterpret_cast<const f32x4_t*>(sp + n0);
+        } else {
+#pragma unroll
+          for (int e = 0; e < 4; ++e)
+            if (n0 + e < N) v[e] = sp[n0 + e];
+        }
+      }
+#pragma unroll
+      for (int e = 0; e < 4; ++e) S[4 * j + e] = v[e];
+    }
+  };
+  float S[G][NPT], Sn[G][NPT];
+#pragma unroll
+  for (int g = 0; g < G; ++g) load(g, S[g]);
+  // step sizes of the wave's 16 channels for all the sequences
+  const int sc = c0 + 16 * wid + ql;
+  const bool sc_ok = sc < inner;
+  const float bias = sc_ok ? dt_bias[sc] : 0.f, dsk = sc_ok ? Dv[sc] : 0.f;
+  const T* wrow = wdt + (size_t)(sc_ok ? sc : 0) * Rp;
+  float dv[4] = {bias, bias, bias, bias};
+  if (sizeof(T) == 2) {
+    f32x4_t acc = f32x4_t{bias, bias, bias, bias};
+    const int r = srow[ql];
+    const T* lrow = low + (size_t)(r < 0 ? 0 : r) * low_ld + 8 * quad;
+#pragma unroll 4
+    for (int k = 0; 32 * k < Rp; ++k) {
+      const bf16x8_t fa = r >= 0 && 32 * k + 8 * quad < R ? *reinterpret_cast<const bf16x8_t*>(lrow + 32 * k)
+                                                          : bf16x8_t{0, 0, 0, 0, 0, 0, 0, 0};
+      acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(fa, *reinterpret_cast<const bf16x8_t*>(wrow + 32 * k + 8 * quad), acc, 0,
+                                                    0, 0);
+    }
+#pragma unroll
+    for (int i = 0; i < 4; ++i) dv[i] = acc[i];
+  } else {
+    for (int k = 0; k < R; ++k) {
+      const float w = lds(wrow + k);
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        const int r = srow[4 * quad + i];
+        dv[i] = fmaf(lds(low + (size_t)(r < 0 ? 0 : r) * low_ld + k), w, dv[i]);
+      }
+    }
+  }
+  float xv[4];
+#pragma unroll
+  for (int i = 0; i < 4; ++i) {
+    const int r = srow[4 * quad + i];
+    xv[i] = r >= 0 && sc_ok ? lds(xc + (size_t)r * inner + sc) : 0.f;
+    const float dt = softplus_hw(dv[i]);
+    sd[4 * quad + i][16 * wid + ql] = f32x2_t{dt * LOG2E, dt * xv[i]};
+  }
+  for (int idx = threadIdx.x; idx < ns * 2 * NP; idx += 256) {
+    const int i = idx / (2 * NP), r = idx - i * 2 * NP, n = r & (NP - 1), row = srow[i];
+    bc[i][r / NP][n] = row >= 0 && n < N ? lds(low + (size_t)row * low_ld + R + (r < NP ? 0 : N) + n) : 0.f;
+  }
+  __syncthreads();
+  for (int i0 = 0; i0 < ns; i0 += G) {
+    if (i0 + G < ns) {
+#pragma unroll
+      for (int g = 0; g < G; ++g) load(i0 + G + g, Sn[g]);
+    }
+#pragma unroll
+    for (int g = 0; g < G; ++g) {
+      const int i = i0 + g;
+      if (i >= ns) break;
+      const f32x2_t d = sd[i][cl];
+      float y = 0.f;
+#pragma unroll
+      for (int j = 0; j < NPT / 4; ++j) {
+        const f32x4_t b4 = *reinterpret_cast<const f32x4_t*>(&bc[i][0][4 * (part + 4 * j)]);
+        const f32x4_t c4 = *reinterpret_cast<const f32x4_t*>(&bc[i][1][4 * (part + 4 * j)]);
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+          S[g][4 * j + e] = fmaf(__builtin_amdgcn_exp2f(d[0] * a2[4 * j + e]), S[g][4 * j + e], d[1] * b4[e]);
+          y = fmaf(S[g][4 * j + e], c4[e], y);
+        }
+      }
+      sy[i][cl] = quad_sum(y);
+      if (ch_ok && sslot[i] >= 0) {
+        float* sp = state + ((size_t)sslot[i] * inner + ch) * N;
+#pragma unroll
+        for (int j = 0; j < NPT / 4; ++j) {
+          const int n0 = 4 * (part + 4 * j);
+          if (n0 >= N) continue;
+          if (vecn) {
+            *reinterpret_cast<f32x4_t*>(sp + n0) = f32x4_t{S[g][4 * j], S[g][4 * j + 1], S[g][4 * j + 2], S[g][4 * j + 3]};
+          } else {
+#pragma unroll
+            for (int e = 0; e < 4; ++e)
+              if (n0 + e < N) sp[n0 + e] = S[g][4 * j + e];
+          }
+        }
+      }
+    }
+#pragma unroll
+    for (int g = 0; g < G; ++g)
+#pragma unroll
+      for (int j = 0; j < NPT; ++j) S[g][j] = Sn[g][j];
+  }
+  __syncthreads();
+#pragma unroll
+  for (int i = 0; i < 4; ++i) {
+    const int r = srow[4 * quad + i];
+    if (r >= 0 && sc_ok) {
+      const float zv = lds(proj + (size_t)r * ld + zoff + sc);
+      sts(out + (size_t)r * inner + sc, fmaf(dsk, xv[i], sy[4 * quad + i][16 * wid + ql]) * silu_t<T>(zv));
+    }
+  }
 }
 
 // ws[seq, c] (chunk c's own contribution) -> the state at the start of chunk c; the slot's state <- the state after the
@@ -489,8 +754,16 @@ GRAG_API hipError_t grag_causal_conv(const void* proj, int ld, int coff, int C, 
   if (grid.y > 65535) return hipErrorInvalidValue;
   const bool one_tile = grid.y == 1;  // every portion in one token tile: the convolution's threads update the pool
   mode = (mode & 3) | (one_tile ? 4 : 0);
+  const uintptr_t amask = dt == 0 ? 7 : 15;
+  const bool vec = C % 4 == 0 && ld % 4 == 0 && coff % 4 == 0 && taps <= 4 && (reinterpret_cast<uintptr_t>(b) & 15) == 0 &&
+                   ((reinterpret_cast<uintptr_t>(proj) | reinterpret_cast<uintptr_t>(cstate) |
+                     reinterpret_cast<uintptr_t>(out)) & amask) == 0;
   DT_DISPATCH(dt, {
-    hipLaunchKernelGGL(causal_conv_kernel<T>, grid, dim3(256), 0, st, (const T*)proj, ld, coff, C, taps, w, b,
+    if (vec)
+      hipLaunchKernelGGL((causal_conv_vec_kernel<T, 4>), dim3((C / 4 + 255) / 256, grid.y, nseq), dim3(256), 0, st,
+                         (const T*)proj, ld, coff, C, taps, w, b, (T*)cstate, slots, q_start, ctx_len, (T*)out, nslots, mode);
+    else
+      hipLaunchKernelGGL(causal_conv_kernel<T>, grid, dim3(256), 0, st, (const T*)proj, ld, coff, C, taps, w, b,
                        (T*)cstate, slots, q_start, ctx_len, (T*)out, nslots, mode);
     if (taps > 1 && !one_tile)
       hipLaunchKernelGGL(conv_state_kernel<T>, dim3((C + 255) / 256, nseq), dim3(256), 0, st, (const T*)proj, ld, coff, C,
@@ -585,7 +858,34 @@ static hipError_t launch_chan_scan(const T* xc, const T* low, int low_ld, const 
   return hipGetLastError();
 }
 
-// chunk_len 0 (or ws / wa null, or max_q_len <= chunk_len): one pass; else the chunk-parallel passes over ws [nseq *
+template <typename T>
+static hipError_t launch_chan_step(const T* xc, const T* low, int low_ld, const T* wdt, int R, int Rp, const float* dt_bias,
+                                   const float* A, const float* Dv, const T* proj, int ld, int zoff, float* state,
+                                   const int* slots, const int* q_start, const int* ctx_len, T* out, int nseq, int inner,
+                                   int N, int nslots, hipStream_t st) {
+  const int tiles = (inner + SC_CH - 1) / SC_CH;
+  int SB = SC_TB;  // sequences per workgroup: as many as leave two workgroups per CU
+  while (SB > 1 && (long)tiles * ((nseq + SB - 1) / SB) < 512) SB >>= 1;
+  const dim3 grid(tiles, (nseq + SB - 1) / SB);
+#define CHAN_STEP(NPT, G)                                                                                              \
+  hipLaunchKernelGGL((chan_step_kernel<T, NPT, G>), grid, dim3(256), 0, st, xc, low, low_ld, wdt, R, Rp, dt_bias, A,   \
+                     Dv, proj, ld, zoff, state, slots, q_start, ctx_len, out, nseq, SB, inner, N, nslots)
+  if (N <= 16) {
+    CHAN_STEP(4, 4);
+  } else if (N <= 32) {
+    CHAN_STEP(8, 2);
+  } else if (N <= 64) {
+    CHAN_STEP(16, 1);
+  } else if (N <= 128) {
+    CHAN_STEP(32, 1);
+  } else {
+    CHAN_STEP(64, 1);
+  }
+#undef CHAN_STEP
+  return hipGetLastError();
+}
+
+// max_q_len 1: decode rows.  chunk_len 0 (or ws / wa null, or max_q_len <= chunk_len): one pass; else the chunk-parallel passes over ws [nseq *
 // ceil(max_q_len / chunk_len)][inner][N] and wa [nseq * chunks][inner] fp32, chunk_len a multiple of 16.
 GRAG_API hipError_t grag_chan_scan(const void* xc, const void* low, int low_ld, const void* wdt, int R, int Rp,
                                    const float* dt_bias, const float* A, const float* Dv, const void* proj, int ld,
@@ -598,6 +898,11 @@ GRAG_API hipError_t grag_chan_scan(const void* xc, const void* low, int low_ld, 
     return hipErrorInvalidValue;
   if (dt == 0 && (low_ld % 8 || (reinterpret_cast<uintptr_t>(low) & 15) || (reinterpret_cast<uintptr_t>(wdt) & 15)))
     return hipErrorInvalidValue;
+  if (max_q_len == 1) {
+    DT_DISPATCH(dt, return (launch_chan_step<T>((const T*)xc, (const T*)low, low_ld, (const T*)wdt, R, Rp, dt_bias, A, Dv,
+                                                (const T*)proj, ld, zoff, state, slots, q_start, ctx_len, (T*)out, nseq,
+                                                inner, N, nslots, st));)
+  }
   if (ws == nullptr || wa == nullptr || chunk_len <= 0 || max_q_len <= chunk_len) {
     DT_DISPATCH(dt, return (launch_chan_scan<T, 0>((const T*)xc, (const T*)low, low_ld, (const T*)wdt, R, Rp, dt_bias, A, Dv,
                                                    (const T*)proj, ld, zoff, state, slots, q_start, ctx_len, (T*)out, nseq,
