@@ -135,17 +135,17 @@ causal_conv_vec_kernel(const T* __restrict__ proj, int ld, int coff, int C, int 
   const T* st = cstate + (size_t)(slot_ok && !fresh ? slot : 0) * (taps - 1) * C + c;
   const T* in = proj + (size_t)qa * ld + coff + c;
   const int nt = min(CONV_TT, qlen - t0), lead = MT - taps;
-  f32x4_t x[MT - 1 + CONV_TT];  // x[MT - 1 + tt] = input of token t0 + tt
+  f32x4_t cur[CONV_TT], win[MT - 1];  // the tile's inputs; the MT - 1 inputs before the one at hand, oldest first
 #pragma unroll
   for (int tt = 0; tt < CONV_TT; ++tt)
-    x[MT - 1 + tt] = tt < nt ? ld4s(in + (size_t)(t0 + tt) * ld) : f32x4_t{0.f, 0.f, 0.f, 0.f};
+    cur[tt] = tt < nt ? ld4s(in + (size_t)(t0 + tt) * ld) : f32x4_t{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
   for (int j = 0; j < MT - 1; ++j) {
-    x[j] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+    win[j] = f32x4_t{0.f, 0.f, 0.f, 0.f};
     const int s = t0 - (MT - 1) + j;  // token index in the portion
     if (j >= lead) {
-      if (s >= 0) x[j] = ld4s(in + (size_t)s * ld);
-      else if (!fresh && slot_ok) x[j] = ld4s(st + (size_t)(taps - 1 + s) * C);
+      if (s >= 0) win[j] = ld4s(in + (size_t)s * ld);
+      else if (!fresh && slot_ok) win[j] = ld4s(st + (size_t)(taps - 1 + s) * C);
     }
   }
   float wt[MT][4];
@@ -156,34 +156,31 @@ causal_conv_vec_kernel(const T* __restrict__ proj, int ld, int coff, int C, int 
   const f32x4_t bias = b ? *reinterpret_cast<const f32x4_t*>(b + c) : f32x4_t{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
   for (int tt = 0; tt < CONV_TT; ++tt) {
-    if (tt >= nt) break;
-    f32x4_t acc = bias;
+    if (tt < nt) {
+      f32x4_t acc = bias;
 #pragma unroll
-    for (int j = 0; j < MT; ++j)
+      for (int j = 0; j < MT - 1; ++j)
 #pragma unroll
-      for (int v = 0; v < 4; ++v) acc[v] = fmaf(wt[j][v], x[tt + j][v], acc[v]);
-    if (!(mode & 1)) {
+        for (int v = 0; v < 4; ++v) acc[v] = fmaf(wt[j][v], win[j][v], acc[v]);
 #pragma unroll
-      for (int v = 0; v < 4; ++v) acc[v] = silu_t<T>(acc[v]);
+      for (int v = 0; v < 4; ++v) acc[v] = fmaf(wt[MT - 1][v], cur[tt][v], acc[v]);
+      if (!(mode & 1)) {
+#pragma unroll
+        for (int v = 0; v < 4; ++v) acc[v] = silu_t<T>(acc[v]);
+      }
+      if (mode & 2) acc += cur[tt];
+      st4s(out + (size_t)(qa + t0 + tt) * C + c, acc);
+#pragma unroll
+      for (int j = 0; j < MT - 2; ++j) win[j] = win[j + 1];
+      win[MT - 2] = cur[tt];
     }
-    if (mode & 2) acc += x[MT - 1 + tt];
-    st4s(out + (size_t)(qa + t0 + tt) * C + c, acc);
   }
   if ((mode & 4) && taps > 1 && index_ok(slot, nslots, ERR_SAMPLER_SLOT)) {  // (t0 is 0: one tile holds the portion)
     T* dst = cstate + (size_t)slot * (taps - 1) * C + c;
 #pragma unroll
     for (int j = 0; j < MT - 1; ++j) {
       if (j < lead) continue;
-      const int s = nt - (MT - 1) + j;  // the token whose input stands at place j after the step
-      f32x4_t v = f32x4_t{0.f, 0.f, 0.f, 0.f};
-      if (s >= 0) {
-        v = ld4s(in + (size_t)s * ld);
-      } else {
-#pragma unroll
-        for (int k = 0; k < MT - 1; ++k)
-          if (k == nt + j) v = x[k];
-      }
-      st4s(dst + (size_t)(j - lead) * C, v);
+      st4s(dst + (size_t)(j - lead) * C, win[j]);
     }
   }
 }
@@ -437,15 +434,51 @@ chan_scan_kernel(const T* __restrict__ xc, const T* __restrict__ low, int low_ld
   // staging role: channel sc of tokens 4 quad + i
   const int sc = c0 + 16 * wid + ql;
   const bool sc_ok = sc < inner;
+  const int scc = sc_ok ? sc : 0;  // (loads of lanes past the last channel or token go to a valid place and are not used)
   const float bias = sc_ok ? dt_bias[sc] : 0.f, dsk = sc_ok ? Dv[sc] : 0.f;
-  const T* wrow = wdt + (size_t)(sc_ok ? sc : 0) * Rp;
-  constexpr int NW = 4;  // matrix fragments kept in registers (R up to 128); the rest is read again per tile
-  bf16x8_t wf[NW];
+  const T* wrow = wdt + (size_t)scc * Rp;
+  constexpr int NW = 8;  // matrix fragments kept in registers (R up to 256); the rest is read again per tile
+  constexpr int NB = NPT <= 8 ? SC_TB * 2 * NP / 256 : 1;  // B / C elements per thread fetched ahead
+  bf16x8_t wf[NW], lf[NW];
+  T xn[4], zn[4], bn[NB];  // (as they are read: nothing waits for them before the walk is over)
   if (sizeof(T) == 2) {
 #pragma unroll
     for (int k = 0; k < NW; ++k)
       wf[k] = 32 * k < Rp ? *reinterpret_cast<const bf16x8_t*>(wrow + 32 * k + 8 * quad) : bf16x8_t{0, 0, 0, 0, 0, 0, 0, 0};
   }
+  // rows of low are padded to a multiple of 8, so a vector that starts below R lies in its row; one that starts past R
+  // meets zeros of the matrix and is taken from the row's start instead
+  auto lfrag = [&](const T* lrow, int k) {
+    return *reinterpret_cast<const bf16x8_t*>(lrow + (32 * k + 8 * quad < R ? 32 * k + 8 * quad : 0));
+  };
+  auto bc_at = [&](int t0, int nb, int idx) {
+    const int t = idx / (2 * NP), r = idx - t * 2 * NP, n = r & (NP - 1);
+    const bool ok = t < nb && n < N;
+    return low[(size_t)(qa + t0 + (ok ? t : 0)) * low_ld + R + (r < NP ? 0 : N) + (ok ? n : 0)];
+  };
+  auto bc_put = [&](int nb, int idx, T v) {  // (past the last token or state number: zeros)
+    (&bc[0][0][0])[idx] = idx / (2 * NP) < nb && (idx & (NP - 1)) < N ? (float)v : 0.f;
+  };
+  auto fetch = [&](int t0) {  // a tile's global reads
+    const int nb = min(SC_TB, qlen - t0);
+    if (sizeof(T) == 2) {
+      const T* lrow = low + (size_t)(qa + t0 + min(ql, nb - 1)) * low_ld;
+#pragma unroll
+      for (int k = 0; k < NW; ++k)
+        if (32 * k < Rp) lf[k] = lfrag(lrow, k);
+    }
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      const size_t row = qa + t0 + min(4 * quad + i, nb - 1);
+      xn[i] = xc[row * inner + scc];
+      if (MODE != 1) zn[i] = proj[row * ld + zoff + scc];
+    }
+    if (NPT <= 8) {
+#pragma unroll
+      for (int u = 0; u < NB; ++u) bn[u] = bc_at(t0, nb, threadIdx.x + 256 * u);
+    }
+  };
+  fetch(0);
   float dtsum = 0.f;
   for (int t0 = 0; t0 < qlen; t0 += SC_TB) {
     const int nb = min(SC_TB, qlen - t0);
@@ -453,73 +486,73 @@ chan_scan_kernel(const T* __restrict__ xc, const T* __restrict__ low, int low_ld
     float dv[4] = {bias, bias, bias, bias};
     if (sizeof(T) == 2) {
       f32x4_t acc = f32x4_t{bias, bias, bias, bias};
-      const T* lrow = low + (size_t)(qa + t0 + (ql < nb ? ql : 0)) * low_ld + 8 * quad;
-      auto frag = [&](int k) {  // (rows are padded to a multiple of 8, so a vector that starts below R lies in its row)
-        return 32 * k + 8 * quad < R ? *reinterpret_cast<const bf16x8_t*>(lrow + 32 * k) : bf16x8_t{0, 0, 0, 0, 0, 0, 0, 0};
-      };
 #pragma unroll
       for (int k = 0; k < NW; ++k)
-        if (32 * k < Rp) acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(frag(k), wf[k], acc, 0, 0, 0);
+        if (32 * k < Rp) acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(lf[k], wf[k], acc, 0, 0, 0);
+      const T* lrow = low + (size_t)(qa + t0 + min(ql, nb - 1)) * low_ld;
       for (int k = NW; 32 * k < Rp; ++k)
-        acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(frag(k), *reinterpret_cast<const bf16x8_t*>(wrow + 32 * k + 8 * quad),
-                                                      acc, 0, 0, 0);
+        acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
+            lfrag(lrow, k), *reinterpret_cast<const bf16x8_t*>(wrow + 32 * k + 8 * quad), acc, 0, 0, 0);
 #pragma unroll
       for (int i = 0; i < 4; ++i) dv[i] = acc[i];
     } else {
       for (int k = 0; k < R; ++k) {
         const float w = lds(wrow + k);
 #pragma unroll
-        for (int i = 0; i < 4; ++i) {
-          const int t = 4 * quad + i;
-          dv[i] = fmaf(lds(low + (size_t)(qa + t0 + (t < nb ? t : 0)) * low_ld + k), w, dv[i]);
-        }
+        for (int i = 0; i < 4; ++i)
+          dv[i] = fmaf(lds(low + (size_t)(qa + t0 + min(4 * quad + i, nb - 1)) * low_ld + k), w, dv[i]);
       }
     }
-    float xv[4];
+    float xv[4], zv[4];
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
-      const int t = 4 * quad + i;
-      xv[i] = (t < nb && sc_ok) ? lds(xc + (size_t)(qa + t0 + t) * inner + sc) : 0.f;
+      xv[i] = (float)xn[i];
+      if (MODE != 1) zv[i] = (float)zn[i];
     }
     __syncthreads();  // the tile before is consumed
+    // (a token past the portion's end leaves the state as it is: dt = 0, B = C = 0)
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
-      const float dt = softplus_hw(dv[i]);
+      const float dt = 4 * quad + i < nb ? softplus_hw(dv[i]) : 0.f;
       sd[4 * quad + i][16 * wid + ql] = f32x2_t{dt * LOG2E, dt * xv[i]};
     }
-    for (int idx = threadIdx.x; idx < nb * 2 * NP; idx += 256) {
-      const int t = idx / (2 * NP), r = idx - t * 2 * NP, n = r & (NP - 1);
-      bc[t][r / NP][n] = n < N ? lds(low + (size_t)(qa + t0 + t) * low_ld + R + (r < NP ? 0 : N) + n) : 0.f;
+    if (NPT <= 8) {
+#pragma unroll
+      for (int u = 0; u < NB; ++u) bc_put(nb, threadIdx.x + 256 * u, bn[u]);
+    } else {
+      for (int idx = threadIdx.x; idx < SC_TB * 2 * NP; idx += 256) bc_put(nb, idx, bc_at(t0, nb, idx));
     }
     __syncthreads();
-#pragma unroll 4
-    for (int t = 0; t < nb; ++t) {
-      const f32x2_t d = sd[t][cl];
-      float y = 0.f;
+    if (t0 + SC_TB < qlen) fetch(t0 + SC_TB);  // in flight during the walk
+    for (int t4 = 0; t4 < nb; t4 += 4) {
 #pragma unroll
-      for (int j = 0; j < NPT / 4; ++j) {
-        const f32x4_t b4 = *reinterpret_cast<const f32x4_t*>(&bc[t][0][4 * (part + 4 * j)]);
+      for (int u = 0; u < 4; ++u) {
+        const int t = t4 + u;
+        const f32x2_t d = sd[t][cl];
+        float y = 0.f;
 #pragma unroll
-        for (int e = 0; e < 4; ++e)
-          S[4 * j + e] = fmaf(__builtin_amdgcn_exp2f(d[0] * a2[4 * j + e]), S[4 * j + e], d[1] * b4[e]);
-        if (MODE != 1) {
-          const f32x4_t c4 = *reinterpret_cast<const f32x4_t*>(&bc[t][1][4 * (part + 4 * j)]);
+        for (int j = 0; j < NPT / 4; ++j) {
+          const f32x4_t b4 = *reinterpret_cast<const f32x4_t*>(&bc[t][0][4 * (part + 4 * j)]);
 #pragma unroll
-          for (int e = 0; e < 4; ++e) y = fmaf(S[4 * j + e], c4[e], y);
+          for (int e = 0; e < 4; ++e)
+            S[4 * j + e] = fmaf(__builtin_amdgcn_exp2f(d[0] * a2[4 * j + e]), S[4 * j + e], d[1] * b4[e]);
+          if (MODE != 1) {
+            const f32x4_t c4 = *reinterpret_cast<const f32x4_t*>(&bc[t][1][4 * (part + 4 * j)]);
+#pragma unroll
+            for (int e = 0; e < 4; ++e) y = fmaf(S[4 * j + e], c4[e], y);
+          }
         }
+        if (MODE == 1) dtsum += d[0];
+        else sy[t][cl] = quad_sum(y);
       }
-      if (MODE == 1) dtsum += d[0];
-      else sy[t][cl] = quad_sum(y);
     }
     if (MODE != 1) {
       __syncthreads();
 #pragma unroll
       for (int i = 0; i < 4; ++i) {
         const int t = 4 * quad + i;
-        if (t < nb && sc_ok) {
-          const float zv = lds(proj + (size_t)(qa + t0 + t) * ld + zoff + sc);
-          sts(out + (size_t)(qa + t0 + t) * inner + sc, fmaf(dsk, xv[i], sy[t][16 * wid + ql]) * silu_t<T>(zv));
-        }
+        const float o = fmaf(dsk, xv[i], sy[t][16 * wid + ql]) * silu_t<T>(zv[i]);
+        if (t < nb && sc_ok) sts(out + (size_t)(qa + t0 + t) * inner + sc, o);
       }
     }
   }
@@ -615,14 +648,17 @@ chan_step_kernel(const T* __restrict__ xc, const T* __restrict__ low, int low_ld
   float dv[4] = {bias, bias, bias, bias};
   if (sizeof(T) == 2) {
     f32x4_t acc = f32x4_t{bias, bias, bias, bias};
-    const int r = srow[ql];
-    const T* lrow = low + (size_t)(r < 0 ? 0 : r) * low_ld + 8 * quad;
-#pragma unroll 4
-    for (int k = 0; 32 * k < Rp; ++k) {
-      const bf16x8_t fa = r >= 0 && 32 * k + 8 * quad < R ? *reinterpret_cast<const bf16x8_t*>(lrow + 32 * k)
-                                                          : bf16x8_t{0, 0, 0, 0, 0, 0, 0, 0};
-      acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(fa, *reinterpret_cast<const bf16x8_t*>(wrow + 32 * k + 8 * quad), acc, 0,
-                                                    0, 0);
+    const T* lrow = low + (size_t)max(srow[ql], 0) * low_ld;
+    for (int k0 = 0; 32 * k0 < Rp; k0 += 4) {  // four fragments of both operands in flight (past R: zeros of the matrix)
+      bf16x8_t fa[4], fb[4];
+#pragma unroll
+      for (int u = 0; u < 4; ++u) {
+        const int o = 32 * (k0 + u) + 8 * quad;
+        fa[u] = *reinterpret_cast<const bf16x8_t*>(lrow + (o < R ? o : 0));
+        fb[u] = o < Rp ? *reinterpret_cast<const bf16x8_t*>(wrow + o) : bf16x8_t{0, 0, 0, 0, 0, 0, 0, 0};
+      }
+#pragma unroll
+      for (int u = 0; u < 4; ++u) acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(fa[u], fb[u], acc, 0, 0, 0);
     }
 #pragma unroll
     for (int i = 0; i < 4; ++i) dv[i] = acc[i];
