@@ -610,7 +610,7 @@ def _vudivik_models(name, dev):
 def _vudivik_kernel_table(dev, H=28, G=4, D=128, W=3584, ff=18944, T=2048, B=64, ctx=2048, bs=16, win=1024, keep=16, N=16,
                           E=16, ident=2, top=4):
     """[(kernel, seconds, bound, fraction of roofline)] for Vudivik's kernels and the like kernels of Leripel (scan,
-    convolution, boundary, router, experts), Pubulix (window attention) and Namudra (normed heads).  The scans are
+    convolution, boundary, router, experts), Pubulix (window attention, rotary store) and Namudra (normed heads).  The scans are
     priced in vector issue slots (2 flops each): per state number and token a scalar-decay scan needs 2 (the two
     multiply-adds), the per-channel one 8 (two products, the exponential at a quarter of the rate, two multiply-adds)."""
     from ..ops.attention import AttnMetadata, sink_attention
@@ -666,7 +666,7 @@ def _vudivik_kernel_table(dev, H=28, G=4, D=128, W=3584, ff=18944, T=2048, B=64,
     add("rope store with biases and head norms", _timed(lambda: rope_vnorm_store(
         proj, 0, H * D, (H + G) * D, pos, tab, meta.slot_mapping, kc, vc, H, G, D, D, D, 1e-6, vnorm=False, bias=bias,
         qw=qw, kw=qw)), bytes_=by)
-    add("leripel rope store", _timed(lambda: rope_vnorm_store(proj, 0, H * D, (H + G) * D, pos, tab, meta.slot_mapping, kc, vc, H, G,
+    add("pubulix rope store", _timed(lambda: rope_vnorm_store(proj, 0, H * D, (H + G) * D, pos, tab, meta.slot_mapping, kc, vc, H, G,
                                                               D, D, D, 1e-6, vnorm=False)), bytes_=by)
     add("namudra qk_norm_store (values are the keys)", _timed(lambda: qk_norm_store(
         proj, 0, H * D, qw, qw, meta.slot_mapping, kc, vc, H, G, D, 1e-6)), bytes_=by)
