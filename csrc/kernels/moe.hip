@@ -1,11 +1,13 @@
 // Mixture-of-experts feed-forward (gfx950) and the residual boundary of layers whose sublayers run side by side:
-//   * router: fp32 logits of a tile of tokens against all experts, softmax scores, group-limited choice of the
-//     best `top` experts per token (a group's score is its best expert's; only the `keep` best groups are open),
-//     the chosen scores as weights (not renormalised); an extra logit row gives the shared expert's sigmoid gate,
+//   * router: fp32 logits of a tile of tokens against all experts, softmax or sigmoid scores, group-limited choice of the
+//     best `top` experts per token (a group's score is that of its best experts; only the `keep` best groups are open),
+//     the chosen scores as weights, as they are or made to sum to a constant; an extra logit row gives the shared
+//     expert's sigmoid gate,
 //   * alignment: the (token, choice) pairs sorted by expert (counting sort in one workgroup),
 //   * grouped GEMMs over the sorted rows: gate | up with the SiLU unit fused, then down, written back in (token,
 //     choice) order,
-//   * boundary: x += mixer + shared * gate + sum_k weight_k expert_k in fp32, then the next RMS norm, one pass;
+//   * boundary: x += mixer + shared * gate + sum_k weight_k expert_k in fp32, then the next RMS norm (or the next two
+//     layer norms, where the sublayers have norms of their own), one pass;
 //   * post-norm boundary: the sublayer's output is RMS-normed before it joins x (and two side-by-side mixers' outputs
 //     are normed apiece before they are added), one pass too.
 // Activations are bf16 or fp32 (dt: 0 = bf16, 1 = fp32); logits, scores, weights and the residual are fp32 in both.
@@ -29,106 +31,120 @@ constexpr int RT_LD = RT_KC + 4;  // LDS row stride (floats): 16-byte rows, bank
 constexpr int RT_MAXR = 256;  // logit rows (experts + the shared gate's row) at most
 constexpr int RT_MAXTOP = 16;
 
-// One token's choice from its logits z [R] (overwritten): scores = softmax of the first E; the `keep` best groups
-// (a group's score is its best expert's) are open; the best `top` experts of the open groups, by falling score, ties
-// to the lower index, weighted by their scores as they are; row E (if any) is the shared expert's gate logit.  With
-// `corr` [E] the choice goes by score + corr (the weights do not).  The last nid of the E rows are identity experts:
-// their weights are summed into idw[t], and the choice's own weight becomes 0 (there is no expert output to weigh).
+// One token's choice from its logits z [R] (in LDS, overwritten), by a whole wave: lane l holds the rows l, l + 64, ...
+// Scores: softmax of the first E logits, or the sigmoid of each.  A group of neighbours counts as much as its `group_top`
+// best experts together; the `keep` best groups are open; the best `top` experts of the open groups, by falling score,
+// ties to the lower index, weighted by their scores as they are or (normed) by scale * score / (sum of the chosen +
+// 1e-20); row E (if any) is the shared expert's gate logit.  With `corr` [E] the choice goes by score + corr (the weights
+// and the groups do not).  The last nid of the E rows are identity experts: their weights are summed into idw[t], and the
+// choice's own weight becomes 0 (there is no expert output to weigh).  All 64 lanes call it with the same arguments; no
+// other wave touches the token's row of z meanwhile.
 struct RouteExtra {
   const float* corr;
   int nid;
   float* idw;
+  int sigmoid, group_top, normed;
+  float scale;
 };
+// the largest v of the wave and its number (ties to the lower one), in every lane; `w` travels along
+__device__ __forceinline__ void wave_best(float& v, float& w, int& e) {
+#pragma unroll
+  for (int o = 32; o > 0; o >>= 1) {
+    const float ov = __shfl_xor(v, o, 64), ow = __shfl_xor(w, o, 64);
+    const int oe = __shfl_xor(e, o, 64);
+    if (ov > v || (ov == v && oe < e)) {
+      v = ov;
+      w = ow;
+      e = oe;
+    }
+  }
+}
 __device__ void route_select(float* z, int E, int R, int top, int ngroups, int keep, int t, int* __restrict__ ids,
                              float* __restrict__ wts, float* __restrict__ sgate, const RouteExtra& rx) {
-  if (R > E && sgate != nullptr) sgate[t] = 1.f / (1.f + expf(-z[E]));
-  float mx = -INFINITY;
-  for (int e = 0; e < E; ++e) mx = fmaxf(mx, z[e]);
-  float sum = 0.f;
-  for (int e = 0; e < E; ++e) sum += expf(z[e] - mx);
-  const float inv = 1.f / sum;
-  // the open groups: `keep` times, the best group not yet taken (by its best logit: softmax keeps the order)
-  const int per = E / ngroups;
-  unsigned long long open_lo = 0, open_hi = 0, open_2 = 0, open_3 = 0;  // bit g: group g is open (up to 256 groups)
-  auto is_open = [&](int g) {
-    const unsigned long long wbits = g < 64 ? open_lo : g < 128 ? open_hi : g < 192 ? open_2 : open_3;
-    return (wbits >> (g & 63)) & 1ull;
-  };
-  for (int n = 0; n < keep; ++n) {
-    int bg = -1;
-    float bv = -INFINITY;
-    for (int g = 0; g < ngroups; ++g) {
-      if (is_open(g)) continue;
-      float gv = -INFINITY;
-      for (int e = g * per; e < (g + 1) * per; ++e) gv = fmaxf(gv, z[e]);
-      if (bg < 0 || gv > bv) {
-        bg = g;
-        bv = gv;
-      }
-    }
-    if (bg < 0) break;
-    const unsigned long long bit = 1ull << (bg & 63);
-    if (bg < 64) open_lo |= bit;
-    else if (bg < 128) open_hi |= bit;
-    else if (bg < 192) open_2 |= bit;
-    else open_3 |= bit;
-  }
-  // the best `top` experts of the open groups; a taken expert's logit is overwritten with -inf
-  float idsum = 0.f;
-  for (int n = 0; n < top; ++n) {
-    int be = -1;
-    float bv = -INFINITY;
-    for (int e = 0; e < E; ++e) {
-      if (!is_open(e / per) || z[e] == -INFINITY) continue;
-      const float v = rx.corr ? fmaf(expf(z[e] - mx), inv, rx.corr[e]) : z[e];
-      if (v > bv || be < 0) {
-        be = e;
-        bv = v;
-      }
-    }
-    if (be < 0) {  // fewer open experts than `top`: the rest of the choices carry no weight
-      ids[(size_t)t * top + n] = 0;
-      wts[(size_t)t * top + n] = 0.f;
-      continue;
-    }
-    ids[(size_t)t * top + n] = be;
-    const float wt = expf(z[be] - mx) * inv;
-    const bool ident = be >= E - rx.nid;
-    wts[(size_t)t * top + n] = ident ? 0.f : wt;
-    if (ident) idsum += wt;
-    z[be] = -INFINITY;
-  }
-  if (rx.idw != nullptr) rx.idw[t] = idsum;
-}
-
-// The same by a whole wave (one group of experts): lane l holds the rows l, l + 64, ... of the logits z, every choice is a
-// wave-wide maximum (ties to the lower index).  All 64 lanes call it with the same arguments.
-__device__ void route_select_wave(const float* z, int E, int R, int top, int t, int* __restrict__ ids,
-                                  float* __restrict__ wts, float* __restrict__ sgate, const RouteExtra& rx) {
   const int lane = threadIdx.x & 63;
   constexpr int PER = RT_MAXR / 64;
   if (lane == 0 && R > E && sgate != nullptr) sgate[t] = 1.f / (1.f + expf(-z[E]));
-  float zl[PER], mx = -INFINITY, sum = 0.f;
+  float zl[PER];
+#pragma unroll
+  for (int j = 0; j < PER; ++j) zl[j] = lane + 64 * j < E ? z[lane + 64 * j] : -INFINITY;
+  if (rx.sigmoid) {
+#pragma unroll
+    for (int j = 0; j < PER; ++j) zl[j] = 1.f / (1.f + expf(-zl[j]));  // (rows past E: 0)
+  } else {
+    float mx = -INFINITY, sum = 0.f;
+#pragma unroll
+    for (int j = 0; j < PER; ++j) mx = fmaxf(mx, zl[j]);
+    mx = wave_max(mx);
+#pragma unroll
+    for (int j = 0; j < PER; ++j) {
+      zl[j] = expf(zl[j] - mx);
+      sum += zl[j];
+    }
+    const float inv = 1.f / wave_sum(sum);
+#pragma unroll
+    for (int j = 0; j < PER; ++j) zl[j] *= inv;
+  }
+  unsigned long long open[4] = {~0ull, ~0ull, ~0ull, ~0ull};  // bit g: group g is open (up to 256 groups)
+  const int per = E / ngroups;
+  if (ngroups > 1) {
+#pragma unroll
+    for (int j = 0; j < PER; ++j) {
+      if (lane + 64 * j < E) z[lane + 64 * j] = zl[j];
+      open[j] = 0;
+    }
+    __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
+    __builtin_amdgcn_wave_barrier();
+    float gv[PER];  // lane l: groups l, l + 64, ...; -inf: none, or already open
+#pragma unroll
+    for (int j = 0; j < PER; ++j) {
+      const int g = lane + 64 * j;
+      gv[j] = -INFINITY;
+      if (g >= ngroups) continue;
+      float sum = 0.f, last = INFINITY;
+      int li = -1;  // the expert counted last
+      for (int n = 0; n < min(rx.group_top, per); ++n) {
+        float bv = -INFINITY;
+        int be = -1;
+        for (int e = g * per; e < (g + 1) * per; ++e) {
+          const float v = z[e];
+          if ((v < last || (v == last && e > li)) && v > bv) {
+            bv = v;
+            be = e;
+          }
+        }
+        if (be < 0) break;
+        sum += bv;
+        last = bv;
+        li = be;
+      }
+      gv[j] = sum;
+    }
+    for (int n = 0; n < keep; ++n) {
+      float bv = -INFINITY, bw = 0.f;
+      int bg = RT_MAXR;
+#pragma unroll
+      for (int j = 0; j < PER; ++j)
+        if (gv[j] > bv) {
+          bv = gv[j];
+          bg = lane + 64 * j;
+        }
+      wave_best(bv, bw, bg);
+#pragma unroll
+      for (int j = 0; j < PER; ++j) {
+        if (bg >> 6 == j) open[j] |= 1ull << (bg & 63);
+        if (bg == lane + 64 * j) gv[j] = -INFINITY;
+      }
+    }
+  }
+  float pick[PER];  // what the choice goes by; -inf: taken, closed, or no row
 #pragma unroll
   for (int j = 0; j < PER; ++j) {
-    zl[j] = lane + 64 * j < E ? z[lane + 64 * j] : -INFINITY;
-    mx = fmaxf(mx, zl[j]);
+    const int e = lane + 64 * j, g = e < E ? e / per : 0;
+    const unsigned long long word = g < 64 ? open[0] : g < 128 ? open[1] : g < 192 ? open[2] : open[3];
+    pick[j] = e < E && ((word >> (g & 63)) & 1ull) ? zl[j] + (rx.corr ? rx.corr[e] : 0.f) : -INFINITY;
   }
-  mx = wave_max(mx);
-#pragma unroll
-  for (int j = 0; j < PER; ++j) {
-    zl[j] = expf(zl[j] - mx);  // (rows past E: 0)
-    sum += zl[j];
-  }
-  const float inv = 1.f / wave_sum(sum);
-  float pick[PER];  // what the choice goes by; -inf: taken, or no row
-#pragma unroll
-  for (int j = 0; j < PER; ++j) {
-    zl[j] *= inv;
-    const int e = lane + 64 * j;
-    pick[j] = e < E ? zl[j] + (rx.corr ? rx.corr[e] : 0.f) : -INFINITY;
-  }
-  float idsum = 0.f;
+  float idsum = 0.f, total = 0.f, mw = 0.f;
+  int mine = 0;  // lane n: choice n and its weight
   for (int n = 0; n < top; ++n) {
     float bv = -INFINITY, bw = 0.f;
     int be = RT_MAXR;
@@ -139,27 +155,25 @@ __device__ void route_select_wave(const float* z, int E, int R, int top, int t, 
         bw = zl[j];
         be = lane + 64 * j;
       }
-#pragma unroll
-    for (int o = 32; o > 0; o >>= 1) {
-      const float ov = __shfl_xor(bv, o, 64), ow = __shfl_xor(bw, o, 64);
-      const int oe = __shfl_xor(be, o, 64);
-      if (ov > bv || (ov == bv && oe < be)) {
-        bv = ov;
-        bw = ow;
-        be = oe;
-      }
-    }
+    wave_best(bv, bw, be);
 #pragma unroll
     for (int j = 0; j < PER; ++j)
       if (be == lane + 64 * j) pick[j] = -INFINITY;
-    const bool none = be >= E, ident = !none && be >= E - rx.nid;
+    const bool none = be >= E;  // fewer open experts than `top`: the rest of the choices carry no weight
+    const bool ident = !none && be >= E - rx.nid;
     if (ident) idsum += bw;
-    if (lane == 0) {
-      ids[(size_t)t * top + n] = none ? 0 : be;
-      wts[(size_t)t * top + n] = none || ident ? 0.f : bw;
+    if (!none) total += bw;
+    if (lane == n) {
+      mine = none ? 0 : be;
+      mw = none || ident ? 0.f : bw;
     }
   }
-  if (lane == 0 && rx.idw != nullptr) rx.idw[t] = idsum;
+  const float mul = rx.normed ? rx.scale / (total + 1e-20f) : 1.f;
+  if (lane < top) {
+    ids[(size_t)t * top + lane] = mine;
+    wts[(size_t)t * top + lane] = mw * mul;
+  }
+  if (lane == 0 && rx.idw != nullptr) rx.idw[t] = idsum * mul;
 }
 
 // h [T][ld] (the normed layer input); wr [R][W] fp32, rows 0 .. E-1 the experts, row E (R = E + 1) the shared expert's
@@ -255,13 +269,8 @@ moe_route_kernel(const T* __restrict__ h, int ld, const float* __restrict__ wr, 
   for (int j = 0; j < RT_MAXR / 16; ++j)
     if (part + 16 * j < R) lgs[tok * (R + 1) + part + 16 * j] = acc[j];
   __syncthreads();
-  if (ngroups == 1) {
-    for (int i = threadIdx.x >> 6; i < RT_TOK && t0 + i < T_; i += 4)
-      route_select_wave(lgs + i * (R + 1), E, R, top, t0 + i, ids, wts, sgate, rx);
-    return;
-  }
-  if (threadIdx.x >= RT_TOK || t0 + threadIdx.x >= T_) return;
-  route_select(lgs + threadIdx.x * (R + 1), E, R, top, ngroups, keep, t0 + threadIdx.x, ids, wts, sgate, rx);
+  for (int i = threadIdx.x >> 6; i < RT_TOK && t0 + i < T_; i += 4)
+    route_select(lgs + i * (R + 1), E, R, top, ngroups, keep, t0 + i, ids, wts, sgate, rx);
 }
 
 // A few tokens (decode rows): one workgroup per token, one wave per logit row (rows w, w + 4, ...), the lanes split the
@@ -306,11 +315,7 @@ moe_route_rows_kernel(const T* __restrict__ h, int ld, const float* __restrict__
     if (lane == 0) z[r] = a;
   }
   __syncthreads();
-  if (ngroups == 1) {
-    if (wid == 0) route_select_wave(z, E, R, top, t, ids, wts, sgate, rx);
-    return;
-  }
-  if (threadIdx.x == 0) route_select(z, E, R, top, ngroups, keep, t, ids, wts, sgate, rx);
+  if (wid == 0) route_select(z, E, R, top, ngroups, keep, t, ids, wts, sgate, rx);
 }
 
 // ------------------------------------------------------------------------------------------------ alignment
@@ -684,17 +689,18 @@ moe_gemm_big_kernel(const bf16* __restrict__ a, int lda, const bf16* __restrict_
 // x [T][H] fp32, in place: x <- keep x + mult * sigmoid(gate + gbias) * (a + bcoef_t b + sum_k ecoef_(t,k) e_(t,k)), every
 // addend optional, the gate too (gate [T][gate_ld] logits in the activation type, gbias [H] fp32)
 // (a, b [T][H]; e [T * K][H], ecoef [T * K]; bcoef [T], null: 1).  Then, each optional: raw [T][raw_ld] <- x in the
-// activation type, out [T][H] <- x / sqrt(mean(x^2) + eps) * w.  grid (T), 256 threads; a thread keeps its elements of
+// activation type, out [T][H] <- x / sqrt(mean(x^2) + eps) * w.  LN: out <- (x - mean) / sqrt(variance + eps) * w and,
+// with w2, out2 <- the same * w2 (the row's deviations are summed in a second pass over the registers).  grid (T), 256 threads; a thread keeps its elements of
 // the row in registers between the sum of squares and the scaling (rows of up to 256 * RB_PER), or re-reads x.
 constexpr int RB_PER = 16;
 
-template <typename T>
+template <typename T, bool LN>
 __global__ void __launch_bounds__(256)
 residual_rmsnorm_kernel(float* __restrict__ x, float keep, const T* __restrict__ a, const T* __restrict__ b,
                         const float* __restrict__ bcoef, const T* __restrict__ e, const float* __restrict__ ecoef,
                         int K, const float* __restrict__ w, float eps, T* __restrict__ out, T* __restrict__ raw,
                         int raw_ld, int H, const T* __restrict__ gate, int gate_ld, const float* __restrict__ gbias,
-                        float mult) {
+                        float mult, const float* __restrict__ w2, T* __restrict__ out2) {
   __shared__ float red[16];
   const size_t t = blockIdx.x, row = t * H;
   const float bc = b ? (bcoef ? bcoef[t] : 1.f) : 0.f;
@@ -735,16 +741,42 @@ residual_rmsnorm_kernel(float* __restrict__ x, float keep, const T* __restrict__
     }
   }
   if (out == nullptr) return;
+  float mean = 0.f;
+  if (LN) {
+    float sum = 0.f;
+    if (fits) {
+#pragma unroll
+      for (int u = 0; u < RB_PER; ++u) sum += v[u];
+    } else {
+      for (int i = threadIdx.x; i < H; i += 256) sum += x[row + i];
+    }
+    mean = block_sum(sum, red) / (float)H;
+    ss = 0.f;
+    if (fits) {
+#pragma unroll
+      for (int u = 0; u < RB_PER; ++u) {
+        v[u] -= mean;
+        if (threadIdx.x + 256 * u < H) ss = fmaf(v[u], v[u], ss);
+      }
+    } else {
+      for (int i = threadIdx.x; i < H; i += 256) ss = fmaf(x[row + i] - mean, x[row + i] - mean, ss);
+    }
+  }
   ss = block_sum(ss, red);
   const float r = 1.f / sqrtf(ss / (float)H + eps);
   if (fits) {
 #pragma unroll
     for (int u = 0; u < RB_PER; ++u) {
       const int i = threadIdx.x + 256 * u;
-      if (i < H) stm(out + row + i, v[u] * r * w[i]);
+      if (i >= H) continue;
+      stm(out + row + i, v[u] * r * w[i]);
+      if (LN && out2) stm(out2 + row + i, v[u] * r * w2[i]);
     }
   } else {
-    for (int i = threadIdx.x; i < H; i += 256) stm(out + row + i, x[row + i] * r * w[i]);
+    for (int i = threadIdx.x; i < H; i += 256) {
+      stm(out + row + i, (x[row + i] - mean) * r * w[i]);
+      if (LN && out2) stm(out2 + row + i, (x[row + i] - mean) * r * w2[i]);
+    }
   }
 }
 
@@ -763,13 +795,13 @@ template <> __device__ __forceinline__ void st4<bf16>(bf16* p, f32x4_t v) {
   *reinterpret_cast<bf16x4_t*>(p) = bf16x4_t{f2bits(v[0]), f2bits(v[1]), f2bits(v[2]), f2bits(v[3])};
 }
 
-template <typename T>
+template <typename T, bool LN>
 __global__ void __launch_bounds__(256)
 residual_rmsnorm_vec_kernel(float* __restrict__ x, float keep, const T* __restrict__ a, const T* __restrict__ b,
                             const float* __restrict__ bcoef, const T* __restrict__ e, const float* __restrict__ ecoef,
                             int K, const float* __restrict__ w, float eps, T* __restrict__ out, T* __restrict__ raw,
                             int raw_ld, int H, const T* __restrict__ gate, int gate_ld,
-                            const float* __restrict__ gbias, float mult) {
+                            const float* __restrict__ gbias, float mult, const float* __restrict__ w2, T* __restrict__ out2) {
   __shared__ float red[16];
   const size_t t = blockIdx.x, row = t * H;
   const float bc = b ? (bcoef ? bcoef[t] : 1.f) : 0.f;
@@ -810,14 +842,33 @@ residual_rmsnorm_vec_kernel(float* __restrict__ x, float keep, const T* __restri
     }
   }
   if (out == nullptr) return;
+  if (LN) {
+    float sum = 0.f;
+#pragma unroll
+    for (int u = 0; u < RBV_PER; ++u) sum += (v[u][0] + v[u][1]) + (v[u][2] + v[u][3]);
+    const float mean = block_sum(sum, red) / (float)H;
+    ss = 0.f;
+#pragma unroll
+    for (int u = 0; u < RBV_PER; ++u) {
+      if ((threadIdx.x + 256 * u) * 4 >= H) continue;
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        v[u][r] -= mean;
+        ss = fmaf(v[u][r], v[u][r], ss);
+      }
+    }
+  }
   ss = block_sum(ss, red);
   const float r = 1.f / sqrtf(ss / (float)H + eps);
 #pragma unroll
   for (int u = 0; u < RBV_PER; ++u) {
     const int i = (threadIdx.x + 256 * u) * 4;
-    if (i < H) {
-      const f32x4_t wv = *reinterpret_cast<const f32x4_t*>(w + i);
-      st4(out + row + i, f32x4_t{v[u][0] * r * wv[0], v[u][1] * r * wv[1], v[u][2] * r * wv[2], v[u][3] * r * wv[3]});
+    if (i >= H) continue;
+    const f32x4_t wv = *reinterpret_cast<const f32x4_t*>(w + i);
+    st4(out + row + i, f32x4_t{v[u][0] * r * wv[0], v[u][1] * r * wv[1], v[u][2] * r * wv[2], v[u][3] * r * wv[3]});
+    if (LN && out2) {
+      const f32x4_t w2v = *reinterpret_cast<const f32x4_t*>(w2 + i);
+      st4(out2 + row + i, f32x4_t{v[u][0] * r * w2v[0], v[u][1] * r * w2v[1], v[u][2] * r * w2v[2], v[u][3] * r * w2v[3]});
     }
   }
 }
@@ -983,12 +1034,13 @@ GRAG_API int grag_moe_max_top() { return RT_MAXTOP; }
 
 GRAG_API hipError_t grag_moe_route(const void* h, int ld, const float* wr, int W, int E, int R, int top, int ngroups,
                                    int keep, int* ids, float* wts, float* sgate, int T_, int dt, const float* corr,
-                                   int nid, float* idw, hipStream_t st) {
-  const RouteExtra rx{corr, nid, idw};
+                                   int nid, float* idw, int sigmoid, int group_top, float scale, int normed,
+                                   hipStream_t st) {
+  const RouteExtra rx{corr, nid, idw, sigmoid, group_top, normed, scale};
   if (T_ <= 0) return hipSuccess;
   if (nid < 0 || nid > E || (nid > 0 && idw == nullptr)) return hipErrorInvalidValue;
   if (E < 1 || R < E || R > RT_MAXR || top < 1 || top > RT_MAXTOP || top > E || ngroups < 1 || E % ngroups ||
-      keep < 1 || keep > ngroups)
+      keep < 1 || keep > ngroups || group_top < 1)
     return hipErrorInvalidValue;
   const size_t bytes = ((size_t)(RT_TOK + R) * RT_LD + (size_t)RT_TOK * (R + 1)) * sizeof(float);
   const int vec = W % 8 == 0 && ld % 8 == 0 && (reinterpret_cast<uintptr_t>(h) & 15) == 0 &&
@@ -1079,26 +1131,42 @@ GRAG_API hipError_t grag_moe_gemm(const void* a, int lda, const void* w, const i
   return hipGetLastError();
 }
 
+template <bool LN>
+static hipError_t launch_residual_norm(float* x, float keep, const void* a, const void* b, const float* bcoef,
+                                       const void* e, const float* ecoef, int K, const float* w, float eps, void* out,
+                                       void* raw, int raw_ld, int T_, int H, int dt, const void* gate, int gate_ld,
+                                       const float* gbias, float mult, const float* w2, void* out2, hipStream_t st) {
+  if (T_ <= 0) return hipSuccess;
+  if (K < 0 || (K > 0 && (e == nullptr || ecoef == nullptr)) || (out != nullptr && w == nullptr) ||
+      (gbias != nullptr && gate == nullptr) || (out2 != nullptr && (w2 == nullptr || out == nullptr)))
+    return hipErrorInvalidValue;
+  auto al16 = [](const void* p) { return (reinterpret_cast<uintptr_t>(p) & 15) == 0; };
+  if (H % 4 == 0 && H <= 4 * 256 * RBV_PER && al16(x) && al16(a) && al16(b) && al16(e) && al16(w) && al16(out) &&
+      al16(raw) && raw_ld % 8 == 0 && al16(gate) && al16(gbias) && gate_ld % 8 == 0 && al16(w2) && al16(out2)) {
+    DT_DISPATCH(dt, hipLaunchKernelGGL((residual_rmsnorm_vec_kernel<T, LN>), dim3(T_), dim3(256), 0, st, x, keep,
+                                       (const T*)a, (const T*)b, bcoef, (const T*)e, ecoef, e ? K : 0, w, eps, (T*)out,
+                                       (T*)raw, raw_ld, H, (const T*)gate, gate_ld, gbias, mult, w2, (T*)out2);)
+    return hipGetLastError();
+  }
+  DT_DISPATCH(dt, hipLaunchKernelGGL((residual_rmsnorm_kernel<T, LN>), dim3(T_), dim3(256), 0, st, x, keep, (const T*)a,
+                                     (const T*)b, bcoef, (const T*)e, ecoef, e ? K : 0, w, eps, (T*)out, (T*)raw,
+                                     raw_ld, H, (const T*)gate, gate_ld, gbias, mult, w2, (T*)out2);)
+  return hipGetLastError();
+}
+
 GRAG_API hipError_t grag_residual_rmsnorm(float* x, float keep, const void* a, const void* b, const float* bcoef,
                                           const void* e, const float* ecoef, int K, const float* w, float eps,
                                           void* out, void* raw, int raw_ld, int T_, int H, int dt, const void* gate,
                                           int gate_ld, const float* gbias, float mult, hipStream_t st) {
-  if (T_ <= 0) return hipSuccess;
-  if (K < 0 || (K > 0 && (e == nullptr || ecoef == nullptr)) || (out != nullptr && w == nullptr) ||
-      (gbias != nullptr && gate == nullptr))
-    return hipErrorInvalidValue;
-  auto al16 = [](const void* p) { return (reinterpret_cast<uintptr_t>(p) & 15) == 0; };
-  if (H % 4 == 0 && H <= 4 * 256 * RBV_PER && al16(x) && al16(a) && al16(b) && al16(e) && al16(w) && al16(out) &&
-      al16(raw) && raw_ld % 8 == 0 && al16(gate) && al16(gbias) && gate_ld % 8 == 0) {
-    DT_DISPATCH(dt, hipLaunchKernelGGL(residual_rmsnorm_vec_kernel<T>, dim3(T_), dim3(256), 0, st, x, keep,
-                                       (const T*)a, (const T*)b, bcoef, (const T*)e, ecoef, e ? K : 0, w, eps, (T*)out,
-                                       (T*)raw, raw_ld, H, (const T*)gate, gate_ld, gbias, mult);)
-    return hipGetLastError();
-  }
-  DT_DISPATCH(dt, hipLaunchKernelGGL(residual_rmsnorm_kernel<T>, dim3(T_), dim3(256), 0, st, x, keep, (const T*)a,
-                                     (const T*)b, bcoef, (const T*)e, ecoef, e ? K : 0, w, eps, (T*)out, (T*)raw,
-                                     raw_ld, H, (const T*)gate, gate_ld, gbias, mult);)
-  return hipGetLastError();
+  return launch_residual_norm<false>(x, keep, a, b, bcoef, e, ecoef, K, w, eps, out, raw, raw_ld, T_, H, dt, gate, gate_ld,
+                                     gbias, mult, nullptr, nullptr, st);
+}
+
+GRAG_API hipError_t grag_residual_layernorm(float* x, const void* a, const void* b, const float* bcoef, const void* e,
+                                            const float* ecoef, int K, const float* w, const float* w2, float eps,
+                                            void* out, void* out2, int T_, int H, int dt, hipStream_t st) {
+  return launch_residual_norm<true>(x, 1.f, a, b, bcoef, e, ecoef, K, w, eps, out, nullptr, 0, T_, H, dt, nullptr, 0,
+                                    nullptr, 1.f, w2, out2, st);
 }
 
 GRAG_API int grag_postnorm_max_width() { return 1024 * PN_PER; }

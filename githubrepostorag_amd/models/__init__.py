@@ -30,6 +30,10 @@ def build_decoder(cfg, **kw):
         from .vudivik import VudivikModel
 
         return VudivikModel(cfg, **kw)
+    if cfg.arch == "kapanex":
+        from .kapanex import KapanexModel
+
+        return KapanexModel(cfg, **kw)
     from .qwen2 import Qwen2Model
 
     return Qwen2Model(cfg, **kw)

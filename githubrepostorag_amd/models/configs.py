@@ -166,6 +166,23 @@ class CappedAttnSpec:
     softcap: float
     rot_dims: int
     rot_base: float
+    qk_unit: bool = False  # q and k are divided by their root mean square per head (no weight)
+
+
+@dataclass(frozen=True)
+class DeltaSpec:
+    """Gated delta rule: ``heads`` heads with an [dim, vdim] fp32 state each, query / key heads shared by
+    heads / kv_heads of them, a causal convolution of ``taps`` taps over q, k and v in front, one decay and one step per
+    head and token, a gated RMS norm per head behind."""
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    taps: int
+
+    @property
+    def conv_channels(self) -> int:
+        return 2 * self.kv_heads * self.dim + self.heads * self.vdim
 
 
 @dataclass(frozen=True)
@@ -247,17 +264,21 @@ class MoESpec:
     unit: str = "glu"  # "glu": gate and up branches; "relu2": one up branch, squared relu
     correction: bool = False  # a learned number per logit row joins the scores that choose, not the weights
     identity: int = 0  # logit rows behind the experts' whose "expert" returns its input
+    score: str = "softmax"  # over the logit rows; "sigmoid": each row by itself
+    group_top: int = 1  # a group of experts counts as much as this many of its best experts together
+    scale: float | None = None  # the chosen scores are made to sum to this (None: weights are the scores as they are)
 
 
 @dataclass(frozen=True)
 class MixerSpec:
-    kind: str  # "parallel" | "mingru" | "retention" | "attention" | "latent_attention" | "mamba2"
+    kind: str  # "parallel" | "mingru" | "retention" | "attention" | "latent_attention" | "mamba2" | "delta"
     left: SinkAttnSpec | NormedAttnSpec | None = None
     right: DecayAttnSpec | SelectiveSSMSpec | None = None
     left_scale: float = 1.0
     right_scale: float = 1.0
     width: int = 0  # mingru state width
-    spec: RetentionSpec | WindowAttnSpec | LatentAttnSpec | ChunkAttnSpec | CappedAttnSpec | SSMSpec | None = None  # single-mixer kinds
+    spec: (RetentionSpec | WindowAttnSpec | LatentAttnSpec | ChunkAttnSpec | CappedAttnSpec | SSMSpec | DeltaSpec
+           | None) = None  # single-mixer kinds
 
 
 @dataclass(frozen=True)
@@ -332,6 +353,20 @@ class HybridConfig:
 
     def param_count(self) -> int:
         H = self.hidden_size
+        if self.arch == "kapanex":
+            n = 2 * self.vocab_size * H + H
+            for L in self.layers:
+                if L.weights_of is not None:
+                    continue
+                m, a, f = L.mixer.kind, L.mixer.spec, L.mlp
+                n += H
+                if m == "delta":
+                    n += a.conv_channels * (H + a.taps) + 2 * a.heads * (H + 1) + a.vdim + 2 * a.heads * a.vdim * H
+                else:
+                    n += H * (a.heads * (a.dim + a.vdim) + a.kv_heads * (a.dim + a.vdim))
+                if f is not None:
+                    n += H + f.experts * (3 * H * f.ff + H) + (3 * H * f.shared_ff + H if f.shared_ff else 0)
+            return n
         if self.arch == "vudivik":
             n = 2 * self.vocab_size * H + H
             for L in self.layers:
@@ -838,6 +873,98 @@ def vudivik_config(name: str, vocab: int, width: int, pattern: str, *, heads: in
                         arch="vudivik", residual_mult=residual_mult)
 
 
+def kapanex_config_from_dict(d: dict, name: str = "kapanex") -> HybridConfig:
+    """The Kapanex design's config.json: a layer list of "delta" / "attention" mixers, each beside an optional
+    mixture-of-experts feed-forward with a norm of its own; a layer may run on another layer's tensors.  Every size and
+    constant is read from it."""
+    layers = []
+    for e in d["layers"]:
+        kind, m = e["type"], e["mixer"]
+        dim = int(m["dim"])
+        if kind == "delta":
+            a = DeltaSpec(int(m["heads"]), int(m.get("kv_heads", m["heads"])), dim, int(m.get("vdim", dim)), int(m["conv"]))
+            if min(a.kv_heads, a.dim, a.vdim, a.taps) < 1 or a.heads % a.kv_heads:
+                raise ValueError(f"bad delta-rule sizes {m}")
+        elif kind == "attention":
+            rot, mask = m.get("rot") or {"dims": 0, "base": 1.0}, m.get("mask") or {}
+            a = CappedAttnSpec(int(m["heads"]), int(m.get("kv_heads", m["heads"])), dim, int(m.get("vdim", dim)),
+                               float(m["scale"]), int(mask.get("size") or 0), 0.0, int(rot["dims"]),
+                               float(rot.get("base", 1.0)), qk_unit=True)
+            if a.heads % a.kv_heads or a.rot_dims % 2 or a.rot_dims > a.dim or a.window < 0:
+                raise ValueError(f"bad attention sizes {m}")
+        else:
+            raise ValueError(f"unknown mixer type {kind!r}")
+        f = e.get("mlp")
+        if f is None:
+            mlp = None
+        elif f.get("kind", "moe") == "moe":
+            r = f["router"]
+            g = r.get("groups") or {"count": 1, "keep": 1}
+            sh = f.get("shared")
+            mlp = MoESpec("moe", int(f["expert"]["ff"]), int(r["experts"]), int(r["top"]), int(g["count"]),
+                          int(g["keep"]), int(sh["ff"]) if sh else 0, score="sigmoid", group_top=2,
+                          scale=float(r.get("scale", 1.0)))
+            if (mlp.groups < 1 or mlp.experts % mlp.groups or not 1 <= mlp.keep <= mlp.groups
+                    or not 1 <= mlp.top <= mlp.keep * (mlp.experts // mlp.groups)):
+                raise ValueError(f"bad router sizes {r}")
+        else:
+            raise ValueError(f"unknown feed-forward kind {f.get('kind')!r}")
+        src = e.get("weights_of")
+        layers.append(HybridLayerSpec(MixerSpec(kind, spec=a), mlp, None if src is None else int(src)))
+    cfg = HybridConfig(name, int(d["vocab"]), int(d["width"]), float(d["norm"]["eps"]), tuple(layers), arch="kapanex",
+                       embed_scale=float((d.get("embedding") or {}).get("scale", 1.0)))
+    for i, L in enumerate(layers):
+        o = cfg.layers[cfg.tensor_layer(i)]
+        if (o.mixer, o.mlp) != (L.mixer, L.mlp):
+            raise ValueError(f"layer {i} differs from layer {L.weights_of}, whose tensors it uses")
+    return cfg
+
+
+def kapanex_config_to_dict(cfg: HybridConfig) -> dict:
+    """Back to the config.json form (checkpoint export, tests)."""
+    layers = []
+    for L in cfg.layers:
+        a, f = L.mixer.spec, L.mlp
+        m = {"heads": a.heads, "kv_heads": a.kv_heads, "dim": a.dim, "vdim": a.vdim}
+        if L.mixer.kind == "delta":
+            m["conv"] = a.taps
+        else:
+            m.update(scale=a.scale, mask={"size": a.window}, rot={"dims": a.rot_dims, "base": a.rot_base})
+        mlp = None if f is None else {
+            "kind": "moe", "expert": {"ff": f.ff}, "shared": {"ff": f.shared_ff} if f.shared_ff else None,
+            "router": {"experts": f.experts, "top": f.top, "scale": f.scale,
+                       "groups": {"count": f.groups, "keep": f.keep}}}
+        e = {"type": L.mixer.kind, "mixer": m, "mlp": mlp}
+        if L.weights_of is not None:
+            e["weights_of"] = L.weights_of
+        layers.append(e)
+    return {"architecture": "Kapanex", "vocab": cfg.vocab_size, "width": cfg.hidden_size, "norm": {"eps": cfg.norm_eps},
+            "embedding": {"scale": cfg.embed_scale}, "layers": layers}
+
+
+def kapanex_config(name: str, vocab: int, width: int, pattern: str, *, heads: int, kv_heads: int, dim: int, ff: int,
+                   window: int = 1024, vdim: int | None = None, rot_dims: int | None = None, delta_heads: int | None = None,
+                   delta_kv_heads: int | None = None, delta_dim: int | None = None, delta_vdim: int | None = None,
+                   taps: int = 4, experts: int = 16, top: int = 4, groups=(4, 2), shared_ff: int = 0,
+                   route_scale: float = 2.0, embed_scale: float | None = None, eps: float = 1e-6, moe: bool = True,
+                   shared: dict | None = None) -> HybridConfig:
+    """A regular Kapanex stack for benches and plumbing tests.  ``pattern``: one letter per layer, d = delta rule,
+    a = window attention; every layer carries the same mixture of experts; ``shared`` {i: j}: layer i runs on layer
+    j's tensors."""
+    mlp = MoESpec("moe", ff, experts, top, groups[0], groups[1], shared_ff, score="sigmoid", group_top=2,
+                  scale=route_scale) if moe else None
+    ddim = delta_dim or dim
+    kinds = {
+        "d": MixerSpec("delta", spec=DeltaSpec(delta_heads or heads, delta_kv_heads or kv_heads, ddim, delta_vdim or ddim,
+                                               taps)),
+        "a": MixerSpec("attention", spec=CappedAttnSpec(heads, kv_heads, dim, vdim or dim, dim ** -0.5, window, 0.0,
+                                                        dim // 2 if rot_dims is None else rot_dims, 1e4, qk_unit=True)),
+    }
+    return HybridConfig(name, vocab, width, eps, tuple(HybridLayerSpec(kinds[c], mlp, (shared or {}).get(i))
+                                                       for i, c in enumerate(pattern)),
+                        arch="kapanex", embed_scale=width ** 0.5 if embed_scale is None else embed_scale)
+
+
 def zofesun_config(name: str, vocab: int, width: int, n_layers: int, *, heads: int, kv_heads: int, dim: int,
                    vdim: int, lin_heads: int, lin_dim: int, lin_vdim: int, ff: int, mingru_every: int = 0,
                    rot_dims: int | None = None, rot_base: float = 10000.0, loop=(0, 0, 1), limit: float = 7.0,
@@ -898,6 +1025,15 @@ HYBRIDS = {
                                    dt_rank=7, taps=3, experts=6, identity=2, top=3, expert_ff=40, shared={3: 0}),
     "vudivik-1b": vudivik_config("vudivik-1b", 32768, 1536, "dmdmdmdm", heads=12, kv_heads=2, dim=128, ff=8960),
     "vudivik-7b": vudivik_config("vudivik-7b", 32768, 3584, "dmdm", heads=28, kv_heads=4, dim=128, ff=18944),
+    # Kapanex: a plumbing-test size and two bench sizes with the layer shapes of a 1.5B / 7B decoder (the routed
+    # experts' active width top * ff plus the shared expert equals the dense decoders' feed-forward width)
+    "kapanex-tiny": kapanex_config("kapanex-tiny", 320, 96, "dadd", heads=4, kv_heads=2, dim=16, vdim=24, window=9,
+                                   rot_dims=8, delta_heads=6, delta_kv_heads=3, delta_dim=8, delta_vdim=12, taps=3,
+                                   experts=6, top=2, groups=(3, 2), ff=40, shared_ff=56, route_scale=1.5, shared={3: 0}),
+    "kapanex-1b": kapanex_config("kapanex-1b", 32768, 1536, "dadadada", heads=12, kv_heads=2, dim=128, ff=1792,
+                                 shared_ff=1792),
+    "kapanex-7b": kapanex_config("kapanex-7b", 32768, 3584, "dada", heads=28, kv_heads=4, dim=128, ff=3840,
+                                 shared_ff=3584),
 }
 
 
@@ -916,6 +1052,8 @@ def config_from_dir(path) -> DecoderConfig | HybridConfig:
         return pubulix_config_from_dict(d, Path(path).name or "pubulix")
     if arch == "vudivik":
         return vudivik_config_from_dict(d, Path(path).name or "vudivik")
+    if arch == "kapanex":
+        return kapanex_config_from_dict(d, Path(path).name or "kapanex")
     mt = str(d.get("model_type", "")).lower()
     if mt == "gpt2":
         return DecoderConfig(Path(path).name, d["vocab_size"], d["n_embd"], d.get("n_inner") or 4 * d["n_embd"],

@@ -109,14 +109,20 @@ _SIGS = {
     "grag_chan_scan_tile": [],
     "grag_chan_scan_max_state": [],
     "grag_chan_scan": [P, P, I, P, I, I, P, P, P, P, I, I, P, P, P, P, P, I, I, I, I, I, P, P, I, I, P],
+    "grag_delta_chunk": [],
+    "grag_delta_max_dim": [],
+    "grag_delta_ws_bytes": [I, I, I],
+    "grag_delta_scan": [P, I, P, I, I, I, P, P, P, P, P, P, P, I, I, I, I, I, I, I, P, P, I, I, P],
+    "grag_delta_step": [P, I, P, I, I, I, I, P, P, P, F, P, P, P, P, P, I, I, I, I, I, I, I, P],
     "grag_moe_max_rows": [],
     "grag_moe_max_top": [],
-    "grag_moe_route": [P, I, P, I, I, I, I, I, I, P, P, P, I, I, P, I, P, P],
+    "grag_moe_route": [P, I, P, I, I, I, I, I, I, P, P, P, I, I, P, I, P, I, I, F, I, P],
     "grag_moe_align": [P, I, I, P, P, P],
     "grag_moe_gemm": [P, I, P, P, P, I, I, I, I, I, P, I, I, I, F, F, F, P, I, P],
     "grag_moe_table_route": [P, P, I, I, I, P, P, I, P],
     "grag_postnorm_max_width": [],
     "grag_postnorm_residual": [P, P, P, P, P, F, P, P, I, P, P, F, F, P, P, I, I, I, P],
+    "grag_residual_layernorm": [P, P, P, P, P, P, I, P, P, F, P, P, I, I, I, P],
     "grag_residual_rmsnorm": [P, F, P, P, P, P, P, I, P, F, P, P, I, I, I, I, P, I, P, F, P],
 }
 
@@ -184,7 +190,7 @@ def call(name: str, *args) -> None:
 
 
 # ---------------------------------------------------------------- device index guard (csrc/kernels/common.h)
-ERR_UNITS = ("norm", "elementwise", "attention", "gemm_tile", "gemm_stream", "seqmix", "gatedmix", "ssm", "moe")
+ERR_UNITS = ("norm", "elementwise", "attention", "gemm_tile", "gemm_stream", "seqmix", "gatedmix", "ssm", "moe", "delta")
 ERR_CODES = {1 << 0: "embed_gather: token id >= vocab", 1 << 1: "qkv_rope_kvstore: KV slot id >= cache slots",
              1 << 2: "qkv_rope_kvstore: position >= RoPE table rows",
              1 << 3: "prefill attention: block-table entry >= KV blocks",

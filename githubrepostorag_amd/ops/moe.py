@@ -4,7 +4,7 @@ top-k choice (or a table that names every token id's experts), and the experts' 
 
 The router's logits, scores and weights are fp32.  The experts run as two grouped GEMMs over the pairs sorted by
 expert; their outputs come back in (token, choice) order and are summed, with the router's weights, in fp32 by the
-layer's residual boundary (ops/norm.py residual_rmsnorm)."""
+layer's residual boundary (ops/norm.py residual_rmsnorm, residual_layernorm)."""
 from __future__ import annotations
 
 import torch
@@ -17,7 +17,8 @@ def _dt(t: torch.Tensor) -> int:
 
 
 def moe_route(h: torch.Tensor, wr: torch.Tensor, E: int, top: int, groups: int = 1, keep: int = 1,
-              corr: torch.Tensor | None = None, identity: int = 0):
+              corr: torch.Tensor | None = None, identity: int = 0, score: str = "softmax", group_top: int = 1,
+              scale: float | None = None):
     """h [T, W]; ``wr`` [R, W] fp32 with the experts' router rows first (R = E, or E + 1 when a last row holds the
     shared expert's gate).  Scores s = softmax of the E logits.  The experts form ``groups`` equal groups of
     neighbours; a group's score is its best expert's, and only experts of the ``keep`` best groups can be chosen.
@@ -25,23 +26,30 @@ def moe_route(h: torch.Tensor, wr: torch.Tensor, E: int, top: int, groups: int =
     gate [T] fp32 = sigmoid of the extra row's logit, or None).
     ``corr`` [E] fp32 joins the scores for the choice only.  ``identity``: the last that many of the E rows are
     identity experts, whose output is the token itself: their ids (>= E - identity) name no expert, their entries of
-    wts are 0, and the third result is instead idw [T] fp32, the sum of their weights."""
+    wts are 0, and the third result is instead idw [T] fp32, the sum of their weights.
+    ``score`` "sigmoid": every expert's score is the sigmoid of its own logit.  ``group_top``: a group's score is the sum
+    of its that many best experts' scores (of all it has, if fewer).  ``scale``: the chosen scores are divided by their
+    sum (+ 1e-20) and multiplied by it."""
     T, W = h.shape
     R = wr.shape[0]
     if identity and (R != E or not 0 < identity <= E):
         raise ValueError("identity experts are the last of the router's rows")
     if E % groups or not 1 <= keep <= groups or not 1 <= top <= E or R not in (E, E + 1):
         raise ValueError("bad router sizes")
+    if score not in ("softmax", "sigmoid") or group_top < 1:
+        raise ValueError("score is 'softmax' or 'sigmoid', and a group has a best expert")
     if not h.is_cuda:
         z = h.float() @ wr.float().T
-        s = torch.softmax(z[:, :E], -1)
-        gs = s.view(T, groups, E // groups).amax(-1)
+        s = torch.softmax(z[:, :E], -1) if score == "softmax" else torch.sigmoid(z[:, :E])
+        gs = s.view(T, groups, E // groups).topk(min(group_top, E // groups), dim=-1).values.sum(-1)
         open_g = torch.zeros(T, groups, dtype=torch.bool)
         open_g.scatter_(1, gs.topk(keep, dim=-1).indices, True)
         closed = ~open_g.repeat_interleave(E // groups, dim=1)
         pick = (s if corr is None else s + corr.float()).masked_fill(closed, -float("inf"))
         ids = pick.sort(dim=-1, descending=True, stable=True).indices[:, :top]
         wts = s.masked_fill(closed, 0.0).gather(1, ids)
+        if scale is not None:
+            wts = wts / (wts.sum(-1, keepdim=True) + 1e-20) * scale
         if identity:
             free = ids >= E - identity
             return ids.to(torch.int32), wts.masked_fill(free, 0.0), (wts * free).sum(-1)
@@ -55,7 +63,8 @@ def moe_route(h: torch.Tensor, wr: torch.Tensor, E: int, top: int, groups: int =
     idw = torch.empty(T, dtype=torch.float32, device=h.device) if identity else None
     assert corr is None or (corr.dtype == torch.float32 and corr.numel() == E and corr.is_contiguous())
     call("grag_moe_route", ptr(h), h.stride(0), ptr(wr), W, E, R, top, groups, keep, ptr(ids), ptr(wts), ptr(gate), T,
-         _dt(h), ptr(corr), identity, ptr(idw))
+         _dt(h), ptr(corr), identity, ptr(idw), 1 if score == "sigmoid" else 0, group_top,
+         0.0 if scale is None else float(scale), 0 if scale is None else 1)
     return ids, wts, idw if identity else gate
 
 

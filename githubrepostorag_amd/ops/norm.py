@@ -279,6 +279,40 @@ def residual_rmsnorm(x: torch.Tensor, a: torch.Tensor | None = None, b: torch.Te
     return out
 
 
+def residual_layernorm(x: torch.Tensor, w: torch.Tensor | None = None, w2: torch.Tensor | None = None, eps: float = 1e-6,
+                       a: torch.Tensor | None = None, b: torch.Tensor | None = None, bcoef: torch.Tensor | None = None,
+                       e: torch.Tensor | None = None, ecoef: torch.Tensor | None = None, out_dtype=torch.bfloat16):
+    """The boundary of a layer whose sublayers read the same ``x`` through norms of their own, one pass over the fp32
+    residual ``x`` [T, H] (updated in place): x <- x + (a + bcoef_t b + sum_k ecoef[t, k] e[t, k]), every addend optional
+    (as in residual_rmsnorm), then with n = (x - mean) / sqrt(variance + eps) over the row returns (n * w, n * w2) in
+    ``out_dtype`` (``w`` / ``w2`` [H] fp32; None where there is no weight)."""
+    assert x.dtype == torch.float32 and x.is_contiguous() and x.dim() == 2 and (w is not None or w2 is None)
+    T, H = x.shape
+    K = 0 if e is None else e.shape[1]
+    if not _on_gpu(x):
+        y = torch.zeros_like(x)
+        if a is not None:
+            y += a.float()
+        if b is not None:
+            y += b.float() * (1.0 if bcoef is None else bcoef.float()[:, None])
+        if e is not None:
+            y += (e.float() * ecoef.float()[:, :, None]).sum(1)
+        x += y
+        c = x - x.mean(-1, keepdim=True)
+        n = c / torch.sqrt(c.pow(2).mean(-1, keepdim=True) + eps)
+        return tuple(None if u is None else (n * u.float()).to(out_dtype) for u in (w, w2))
+    for t in (a, b):
+        assert t is None or (t.dtype == out_dtype and t.is_contiguous() and t.shape == (T, H))
+    assert e is None or (e.dtype == out_dtype and e.is_contiguous() and e.shape == (T, K, H)
+                         and ecoef.dtype == torch.float32 and ecoef.is_contiguous() and ecoef.shape == (T, K))
+    assert bcoef is None or (bcoef.dtype == torch.float32 and bcoef.numel() == T)
+    assert all(u is None or (u.dtype == torch.float32 and u.is_contiguous() and u.numel() == H) for u in (w, w2))
+    outs = [None if u is None else torch.empty(T, H, dtype=out_dtype, device=x.device) for u in (w, w2)]
+    call("grag_residual_layernorm", ptr(x), ptr(a), ptr(b), ptr(bcoef), ptr(e), ptr(ecoef), K, ptr(w), ptr(w2), float(eps),
+         ptr(outs[0]), ptr(outs[1]), T, H, 0 if out_dtype == torch.bfloat16 else 1)
+    return tuple(outs)
+
+
 # ---------------------------------------------------------------------------------------------- post-norm boundary
 def postnorm_residual(x: torch.Tensor, a: torch.Tensor | None = None, wa: torch.Tensor | None = None,
                       b: torch.Tensor | None = None, wb: torch.Tensor | None = None, bscale: float = 1.0,

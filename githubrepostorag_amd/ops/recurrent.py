@@ -1,5 +1,6 @@
 """Recurrent sequence mixers with a carried fp32 state per sequence (HIP on device tensors, plain fp32 loops on
-CPU): linear attention with a fixed per-head decay, and the minGRU gated recurrence.
+CPU): linear attention with a fixed per-head decay, the minGRU gated recurrence, state-space scans, and the gated delta
+rule.
 
 State lives in slot-indexed pools ([slots, ...] fp32) owned by the engine; ``meta.state_slots`` [nseq] names each
 sequence's slot.  A sequence whose first token of the step is position 0 starts from a zero state (so a freed
@@ -329,3 +330,80 @@ def _selective_scan_cpu(x, low, wdt, dt_bias, A, skip, z, state, m, out):
             S = torch.exp(dt[t, :, None] * A) * S + (dt[t] * x[t])[:, None] * B[t]
             out[t] = ((S @ C[t] + skip.float() * x[t]) * g[t]).to(out.dtype)
         state[sl[s]] = S
+
+
+# ---------------------------------------------------------------------------------------------- gated delta rule
+def _delta_ws(m: AttnMetadata, rows: int, H: int, G: int, d: int, dt: int, device):
+    """Scratch of the chunked delta rule: per 64-token chunk the operands the scan reads (see grag_delta_scan).  A
+    sequence's chunks start at row (its first token) // chunk + (its number), so unequal portions waste nothing."""
+    chunk = lib().grag_delta_chunk()
+    n = rows // chunk + m.num_seqs
+    kb = lib().grag_delta_ws_bytes(d, dt, 0)
+    hb = lib().grag_delta_ws_bytes(d, dt, 1)
+    return (torch.empty(n * G * kb, dtype=torch.uint8, device=device),
+            torch.empty(n * H * hb, dtype=torch.uint8, device=device), n)
+
+
+def gated_delta(xc: torch.Tensor, proj: torch.Tensor, boff: int, aoff: int, goff: int, a_log: torch.Tensor,
+                dt_bias: torch.Tensor, w: torch.Tensor, eps: float, state: torch.Tensor, meta: AttnMetadata, H: int, G: int,
+                d: int, vd: int) -> torch.Tensor:
+    """Gated delta rule.  ``xc`` [T, 2 G d + H vd] (the convolution's output): q heads (G x d) | k heads | v heads (H x
+    vd); columns boff / aoff (H each) and goff (H vd) of the fused projection ``proj``: the steps', the decays' and the
+    output gate's raw values.  q and k become unit vectors, x / sqrt(sum x^2 + 1e-6), q times d^-1/2.  Per head h (q / k
+    head h // (H / G)), in fp32 with the state S [slots, H, d, vd]:
+        g = exp(-exp(a_log[h]) softplus(a + dt_bias[h])),  beta = sigmoid(b)
+        S <- g S;  u = beta (v - S^T k);  S <- S + k u^T;  o = S^T q
+    Returns o / sqrt(mean(o^2) + eps) * w * silu(gate) per head, [T, H vd] in xc's dtype (``w`` [H vd] fp32)."""
+    T, C = xc.shape
+    assert C == 2 * G * d + H * vd and H % G == 0
+    y = torch.empty(T, H * vd, dtype=xc.dtype, device=xc.device)
+    for m, r0, r1 in _parts(meta):
+        if r1 <= r0:
+            continue
+        x, p = xc[r0:r1], proj[r0:r1]
+        if not xc.is_cuda:
+            _gated_delta_cpu(x.float(), p, boff, aoff, goff, a_log, dt_bias, w, eps, state, m, H, G, d, vd, y[r0:r1])
+            continue
+        assert xc.is_contiguous() and proj.stride(1) == 1 and xc.dtype == proj.dtype
+        assert state.dtype == torch.float32 and state.is_contiguous() and state.shape[1:] == (H, d, vd)
+        assert all(t.dtype == torch.float32 and t.is_contiguous() for t in (a_log, dt_bias, w))
+        assert a_log.numel() == H and dt_bias.numel() == H and w.numel() == H * vd
+        assert max(boff + H, aoff + H, goff + H * vd) <= proj.shape[1]
+        if max(d, vd) > lib().grag_delta_max_dim():
+            raise ValueError(f"the delta-rule kernels hold head sizes of up to {lib().grag_delta_max_dim()}")
+        tail = (ptr(state), ptr(m.state_slots), ptr(m.q_start), ptr(m.ctx_len))
+        if m.max_q_len == 1:  # decode rows: the step and the gated norm in one kernel
+            call("grag_delta_step", ptr(x), C, ptr(p), proj.stride(0), boff, aoff, goff, ptr(a_log), ptr(dt_bias), ptr(w),
+                 float(eps), *tail, ptr(y[r0:r1]), m.num_seqs, H, G, d, vd, state.shape[0], _dt(xc))
+            continue
+        wk, wh, nchunks = _delta_ws(m, r1 - r0, H, G, d, _dt(xc), xc.device)
+        o = torch.empty(r1 - r0, H * vd, dtype=torch.float32, device=xc.device)
+        call("grag_delta_scan", ptr(x), C, ptr(p), proj.stride(0), boff, aoff, ptr(a_log), ptr(dt_bias), *tail, ptr(o),
+             m.num_seqs, H, G, d, vd, state.shape[0], _dt(xc), ptr(wk), ptr(wh), nchunks, m.max_q_len)
+        gated_rmsnorm(o, w, p, goff, eps, y[r0:r1], groups=H, gate="silu")
+    return y
+
+
+def _gated_delta_cpu(x, p, boff, aoff, goff, a_log, dt_bias, w, eps, state, m, H, G, d, vd, y):
+    F = torch.nn.functional
+    qs, cl, sl = m.q_start.tolist(), m.ctx_len.tolist(), m.state_slots.tolist()
+    unit = lambda t: t / torch.sqrt(t.pow(2).sum(-1, keepdim=True) + 1e-6)
+    q = (unit(x[:, :G * d].reshape(-1, G, d)) * d ** -0.5).repeat_interleave(H // G, dim=1)
+    k = unit(x[:, G * d:2 * G * d].reshape(-1, G, d)).repeat_interleave(H // G, dim=1)
+    v = x[:, 2 * G * d:].reshape(-1, H, vd)
+    beta = torch.sigmoid(p[:, boff:boff + H].float())
+    raw = p[:, aoff:aoff + H].float() + dt_bias.float()
+    g = torch.exp(-torch.exp(a_log.float()) * F.softplus(raw, threshold=20.0))
+    o = torch.zeros(x.shape[0], H, vd)
+    for s in range(m.num_seqs):
+        a, e = qs[s], qs[s + 1]
+        if e <= a:
+            continue
+        S = torch.zeros(H, d, vd) if cl[s] - (e - a) == 0 else state[sl[s]].clone()
+        for t in range(a, e):
+            S = g[t, :, None, None] * S
+            u = beta[t, :, None] * (v[t] - (S * k[t, :, :, None]).sum(1))
+            S = S + k[t, :, :, None] * u[:, None, :]
+            o[t] = (S * q[t, :, :, None]).sum(1)
+        state[sl[s]] = S
+    gated_rmsnorm(o.reshape(-1, H * vd), w, p, goff, eps, y, groups=H, gate="silu")
