@@ -134,8 +134,8 @@ delta_prep_kernel(const T* __restrict__ xc, int C, const T* __restrict__ proj, i
   const int ND = (d + 31) / 32, dp = 32 * ND, lk = dp + (sizeof(T) == 2 ? 8 : 4);
   T* Ks = reinterpret_cast<T*>(dsm);
   T* Qs = Ks + DC * lk;
-  float* Ts = reinterpret_cast<float*>(Qs + DC * lk);  // [64][68]
-  float* Af = Ts + DC * 68;                            // [10][64][4]
+  float* Ts = reinterpret_cast<float*>(dsm);  // [64][68], in the place of K and Q once they have been used
+  float* Af = Ts + max(DC * 68, 2 * DC * lk * (int)sizeof(T) / 4);  // [10][64][4]
   float* rk = Af + 2560;                               // [64] each: 1 / |k|, d^-1/2 / |q|, L (two parts), beta
   float *rq = rk + DC, *lh = rq + DC, *ll = lh + DC, *be = ll + DC;
   const int lane = threadIdx.x & 63, w = threadIdx.x >> 6, ql = lane & 15, quad = lane >> 4;
@@ -462,7 +462,7 @@ delta_scan_kernel(const T* __restrict__ xc, int C, float* __restrict__ state, co
 }
 
 // ------------------------------------------------------------------------------------------------ one token
-// grid (H, nseq), NT threads: a thread holds V columns of the rows rg, rg + RG, ... (at most RPT of them) of its head's
+// grid (H, nseq), up to NT threads: a thread holds V columns of the rows rg, rg + RG, ... (at most RPT of them) of its head's
 // state, ncp = 2^n >= vd / V threads a row, RG = NT / ncp row groups.  The state is read once and written once; S^T k and
 // S^T q are sums over the row groups.  Then y = o / rms(o) * w * silu(gate).
 template <int V> __device__ __forceinline__ void ldV(const float* p, float (&v)[V]) {
@@ -479,8 +479,8 @@ template <int V> __device__ __forceinline__ void stV(float* p, const float (&v)[
   else *p = v[0];
 }
 
-template <typename T, int V, int RPT>
-__global__ void __launch_bounds__(1024)
+template <typename T, int V, int RPT, int NT>
+__global__ void __launch_bounds__(NT)
 delta_step_kernel(const T* __restrict__ xc, int C, const T* __restrict__ proj, int ld, int boff, int aoff, int goff,
                   const float* __restrict__ a_log, const float* __restrict__ dt_bias, const float* __restrict__ wn,
                   float eps, float* __restrict__ state, const int* __restrict__ slots, const int* __restrict__ q_start,
@@ -630,7 +630,8 @@ GRAG_API hipError_t grag_delta_scan(const void* xc, int C, const void* proj, int
   const int ND = (d + 31) / 32, dp = 32 * ND;
   const int vec = C % 8 == 0 && d % 8 == 0 && (reinterpret_cast<uintptr_t>(xc) & 15) == 0;
   const size_t lk = dp + (dt == 0 ? 8 : 4);
-  const size_t bytes = 2 * DC * lk * (dt == 0 ? 2 : 4) + (DC * 68 + 2560 + 5 * DC) * sizeof(float);
+  const size_t kq = 2 * DC * lk * (dt == 0 ? 2 : 4), tri = DC * 68 * sizeof(float);
+  const size_t bytes = (kq > tri ? kq : tri) + (2560 + 5 * DC) * sizeof(float);
 #define DELTA_SCAN(NDM)                                                                                              \
   hipLaunchKernelGGL((delta_scan_kernel<T, NDM>), grid, dim3(256), 0, st, (const T*)xc, C, state, slots, q_start,    \
                      ctx_len, out, H, G, d, vd, nslots, (const T*)wk, (const float*)wh, nchunks)
@@ -668,20 +669,23 @@ GRAG_API hipError_t grag_delta_step(const void* xc, int C, const void* proj, int
   while (ncp * V < vd) ncp <<= 1;
   while ((d + nt / ncp - 1) / (nt / ncp) > maxr) nt <<= 1;  // (at most 1024: 256 x 256 numbers are 64 a thread)
   const int rpt = (d + nt / ncp - 1) / (nt / ncp);
-#define DELTA_STEP(VV, RPT)                                                                                           \
-  hipLaunchKernelGGL((delta_step_kernel<T, VV, RPT>), dim3(H, nseq), dim3(nt), 0, st, (const T*)xc, C, (const T*)proj, \
+#define DELTA_STEP(VV, RPT, NT)                                                                                       \
+  hipLaunchKernelGGL((delta_step_kernel<T, VV, RPT, NT>), dim3(H, nseq), dim3(nt), 0, st, (const T*)xc, C, (const T*)proj, \
                      ld, boff, aoff, goff, a_log, dt_bias, wn, eps, state, slots, q_start, ctx_len, (T*)y, H, G, d, vd, \
                      nslots, ncp)
   DT_DISPATCH(dt, {
     if (V == 1) {
-      if (rpt <= 16) DELTA_STEP(1, 16);
-      else DELTA_STEP(1, 64);
+      if (nt > 256) DELTA_STEP(1, 64, 1024);
+      else if (rpt <= 16) DELTA_STEP(1, 16, 256);
+      else DELTA_STEP(1, 64, 256);
+    } else if (nt > 256) {
+      DELTA_STEP(4, 16, 1024);
     } else if (rpt <= 4) {
-      DELTA_STEP(4, 4);
+      DELTA_STEP(4, 4, 256);
     } else if (rpt <= 8) {
-      DELTA_STEP(4, 8);
+      DELTA_STEP(4, 8, 256);
     } else {
-      DELTA_STEP(4, 16);
+      DELTA_STEP(4, 16, 256);
     }
   })
 #undef DELTA_STEP

@@ -31,14 +31,15 @@ constexpr int RT_LD = RT_KC + 4;  // LDS row stride (floats): 16-byte rows, bank
 constexpr int RT_MAXR = 256;  // logit rows (experts + the shared gate's row) at most
 constexpr int RT_MAXTOP = 16;
 
-// One token's choice from its logits z [R] (in LDS, overwritten), by a whole wave: lane l holds the rows l, l + 64, ...
+// One token's choice from its logits z [R] (in LDS, overwritten), by SW = 16, 32 or 64 neighbouring lanes (SW >= E, or 64):
+// lane l of them holds the rows l, l + SW, ...
 // Scores: softmax of the first E logits, or the sigmoid of each.  A group of neighbours counts as much as its `group_top`
 // best experts together; the `keep` best groups are open; the best `top` experts of the open groups, by falling score,
 // ties to the lower index, weighted by their scores as they are or (normed) by scale * score / (sum of the chosen +
 // 1e-20); row E (if any) is the shared expert's gate logit.  With `corr` [E] the choice goes by score + corr (the weights
 // and the groups do not).  The last nid of the E rows are identity experts: their weights are summed into idw[t], and the
-// choice's own weight becomes 0 (there is no expert output to weigh).  All 64 lanes call it with the same arguments; no
-// other wave touches the token's row of z meanwhile.
+// choice's own weight becomes 0 (there is no expert output to weigh).  All SW lanes call it with the same arguments; nobody
+// else touches the token's row of z meanwhile.
 struct RouteExtra {
   const float* corr;
   int nid;
@@ -46,10 +47,10 @@ struct RouteExtra {
   int sigmoid, group_top, normed;
   float scale;
 };
-// the largest v of the wave and its number (ties to the lower one), in every lane; `w` travels along
-__device__ __forceinline__ void wave_best(float& v, float& w, int& e) {
+// the largest v of SW lanes and its number (ties to the lower one), in every lane; `w` travels along
+template <int SW> __device__ __forceinline__ void best_of(float& v, float& w, int& e) {
 #pragma unroll
-  for (int o = 32; o > 0; o >>= 1) {
+  for (int o = SW / 2; o > 0; o >>= 1) {
     const float ov = __shfl_xor(v, o, 64), ow = __shfl_xor(w, o, 64);
     const int oe = __shfl_xor(e, o, 64);
     if (ov > v || (ov == v && oe < e)) {
@@ -59,14 +60,15 @@ __device__ __forceinline__ void wave_best(float& v, float& w, int& e) {
     }
   }
 }
+template <int SW>
 __device__ void route_select(float* z, int E, int R, int top, int ngroups, int keep, int t, int* __restrict__ ids,
                              float* __restrict__ wts, float* __restrict__ sgate, const RouteExtra& rx) {
-  const int lane = threadIdx.x & 63;
-  constexpr int PER = RT_MAXR / 64;
+  const int lane = threadIdx.x & (SW - 1);
+  constexpr int PER = SW == 64 ? RT_MAXR / 64 : 1;
   if (lane == 0 && R > E && sgate != nullptr) sgate[t] = 1.f / (1.f + expf(-z[E]));
   float zl[PER];
 #pragma unroll
-  for (int j = 0; j < PER; ++j) zl[j] = lane + 64 * j < E ? z[lane + 64 * j] : -INFINITY;
+  for (int j = 0; j < PER; ++j) zl[j] = lane + SW * j < E ? z[lane + SW * j] : -INFINITY;
   if (rx.sigmoid) {
 #pragma unroll
     for (int j = 0; j < PER; ++j) zl[j] = 1.f / (1.f + expf(-zl[j]));  // (rows past E: 0)
@@ -74,13 +76,16 @@ __device__ void route_select(float* z, int E, int R, int top, int ngroups, int k
     float mx = -INFINITY, sum = 0.f;
 #pragma unroll
     for (int j = 0; j < PER; ++j) mx = fmaxf(mx, zl[j]);
-    mx = wave_max(mx);
+#pragma unroll
+    for (int o = SW / 2; o > 0; o >>= 1) mx = fmaxf(mx, __shfl_xor(mx, o, 64));
 #pragma unroll
     for (int j = 0; j < PER; ++j) {
       zl[j] = expf(zl[j] - mx);
       sum += zl[j];
     }
-    const float inv = 1.f / wave_sum(sum);
+#pragma unroll
+    for (int o = SW / 2; o > 0; o >>= 1) sum += __shfl_xor(sum, o, 64);
+    const float inv = 1.f / sum;
 #pragma unroll
     for (int j = 0; j < PER; ++j) zl[j] *= inv;
   }
@@ -89,15 +94,15 @@ __device__ void route_select(float* z, int E, int R, int top, int ngroups, int k
   if (ngroups > 1) {
 #pragma unroll
     for (int j = 0; j < PER; ++j) {
-      if (lane + 64 * j < E) z[lane + 64 * j] = zl[j];
-      open[j] = 0;
+      if (lane + SW * j < E) z[lane + SW * j] = zl[j];
     }
+    open[0] = open[1] = open[2] = open[3] = 0;
     __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
     __builtin_amdgcn_wave_barrier();
-    float gv[PER];  // lane l: groups l, l + 64, ...; -inf: none, or already open
+    float gv[PER];  // lane l: groups l, l + SW, ...; -inf: none, or already open
 #pragma unroll
     for (int j = 0; j < PER; ++j) {
-      const int g = lane + 64 * j;
+      const int g = lane + SW * j;
       gv[j] = -INFINITY;
       if (g >= ngroups) continue;
       float sum = 0.f, last = INFINITY;
@@ -126,20 +131,21 @@ __device__ void route_select(float* z, int E, int R, int top, int ngroups, int k
       for (int j = 0; j < PER; ++j)
         if (gv[j] > bv) {
           bv = gv[j];
-          bg = lane + 64 * j;
+          bg = lane + SW * j;
         }
-      wave_best(bv, bw, bg);
+      best_of<SW>(bv, bw, bg);
 #pragma unroll
-      for (int j = 0; j < PER; ++j) {
+      for (int j = 0; j < 4; ++j)
         if (bg >> 6 == j) open[j] |= 1ull << (bg & 63);
-        if (bg == lane + 64 * j) gv[j] = -INFINITY;
-      }
+#pragma unroll
+      for (int j = 0; j < PER; ++j)
+        if (bg == lane + SW * j) gv[j] = -INFINITY;
     }
   }
   float pick[PER];  // what the choice goes by; -inf: taken, closed, or no row
 #pragma unroll
   for (int j = 0; j < PER; ++j) {
-    const int e = lane + 64 * j, g = e < E ? e / per : 0;
+    const int e = lane + SW * j, g = e < E ? e / per : 0;
     const unsigned long long word = g < 64 ? open[0] : g < 128 ? open[1] : g < 192 ? open[2] : open[3];
     pick[j] = e < E && ((word >> (g & 63)) & 1ull) ? zl[j] + (rx.corr ? rx.corr[e] : 0.f) : -INFINITY;
   }
@@ -153,12 +159,12 @@ __device__ void route_select(float* z, int E, int R, int top, int ngroups, int k
       if (pick[j] > bv) {
         bv = pick[j];
         bw = zl[j];
-        be = lane + 64 * j;
+        be = lane + SW * j;
       }
-    wave_best(bv, bw, be);
+    best_of<SW>(bv, bw, be);
 #pragma unroll
     for (int j = 0; j < PER; ++j)
-      if (be == lane + 64 * j) pick[j] = -INFINITY;
+      if (be == lane + SW * j) pick[j] = -INFINITY;
     const bool none = be >= E;  // fewer open experts than `top`: the rest of the choices carry no weight
     const bool ident = !none && be >= E - rx.nid;
     if (ident) idsum += bw;
@@ -175,6 +181,10 @@ __device__ void route_select(float* z, int E, int R, int top, int ngroups, int k
   }
   if (lane == 0 && rx.idw != nullptr) rx.idw[t] = idsum * mul;
 }
+
+template <int N> struct Lanes {
+  static constexpr int value = N;
+};
 
 // h [T][ld] (the normed layer input); wr [R][W] fp32, rows 0 .. E-1 the experts, row E (R = E + 1) the shared expert's
 // gate.  ids [T][top] int32, wts [T][top] fp32 (the chosen experts by falling score; ties to the lower index),
@@ -269,8 +279,14 @@ moe_route_kernel(const T* __restrict__ h, int ld, const float* __restrict__ wr, 
   for (int j = 0; j < RT_MAXR / 16; ++j)
     if (part + 16 * j < R) lgs[tok * (R + 1) + part + 16 * j] = acc[j];
   __syncthreads();
-  for (int i = threadIdx.x >> 6; i < RT_TOK && t0 + i < T_; i += 4)
-    route_select(lgs + i * (R + 1), E, R, top, ngroups, keep, t0 + i, ids, wts, sgate, rx);
+  auto select = [&](auto sw) {
+    constexpr int SW = decltype(sw)::value;
+    for (int i = threadIdx.x / SW; i < RT_TOK && t0 + i < T_; i += 256 / SW)
+      route_select<SW>(lgs + i * (R + 1), E, R, top, ngroups, keep, t0 + i, ids, wts, sgate, rx);
+  };
+  if (E <= 16) select(Lanes<16>());
+  else if (E <= 32) select(Lanes<32>());
+  else select(Lanes<64>());
 }
 
 // A few tokens (decode rows): one workgroup per token, one wave per logit row (rows w, w + 4, ...), the lanes split the
@@ -315,7 +331,11 @@ moe_route_rows_kernel(const T* __restrict__ h, int ld, const float* __restrict__
     if (lane == 0) z[r] = a;
   }
   __syncthreads();
-  if (wid == 0) route_select(z, E, R, top, ngroups, keep, t, ids, wts, sgate, rx);
+  if (E <= 16) {
+    if (threadIdx.x < 16) route_select<16>(z, E, R, top, ngroups, keep, t, ids, wts, sgate, rx);
+  } else if (wid == 0) {
+    route_select<64>(z, E, R, top, ngroups, keep, t, ids, wts, sgate, rx);
+  }
 }
 
 // ------------------------------------------------------------------------------------------------ alignment

@@ -1272,6 +1272,49 @@ gated_rmsnorm_wave_kernel(const float* __restrict__ x, const float* __restrict__
   }
 }
 
+// the same in accesses of four columns (N a multiple of 4, N <= 256, aligned rows): LG lanes a group, LG = 2^n >= N / 4,
+// (token, group) pairs in a row.  grid (ceil(T * groups * LG / 256)).
+template <typename T, int LG>
+__global__ void __launch_bounds__(256)
+gated_rmsnorm_vec_kernel(const float* __restrict__ x, const float* __restrict__ w, const T* __restrict__ proj, int ld,
+                         int goff, T* __restrict__ out, int out_ld, int T_, int N, int groups, float eps, float out_scale,
+                         int silu_gate) {
+  const long pair = ((long)blockIdx.x * 256 + threadIdx.x) / LG;
+  const int i = threadIdx.x % LG * 4;
+  const bool on = pair < (long)T_ * groups && i < N;
+  const int t = on ? (int)(pair / groups) : 0, c0 = on ? (int)(pair - (long)t * groups) * N + i : 0;
+  const bool first = silu_gate & 2;
+  f32x4_t v = f32x4_t{0.f, 0.f, 0.f, 0.f}, gt = v;
+  if (on) {
+    v = *reinterpret_cast<const f32x4_t*>(x + (size_t)t * N * groups + c0);
+    if (sizeof(T) == 2) {
+      const bf16x4_t g = *reinterpret_cast<const bf16x4_t*>(proj + (size_t)t * ld + goff + c0);
+      gt = f32x4_t{bits2f(g[0]), bits2f(g[1]), bits2f(g[2]), bits2f(g[3])};
+    } else {
+      gt = *reinterpret_cast<const f32x4_t*>(proj + (size_t)t * ld + goff + c0);
+    }
+  }
+  float ss = 0.f;
+#pragma unroll
+  for (int e = 0; e < 4; ++e) {
+    gt[e] = (silu_gate & 1) ? silu_acc(gt[e]) : sigmoid_acc(gt[e]);
+    const float u = first ? v[e] * gt[e] : v[e];
+    ss = fmaf(u, u, ss);
+  }
+#pragma unroll
+  for (int o = LG / 2; o > 0; o >>= 1) ss += __shfl_xor(ss, o, 64);
+  if (!on) return;
+  const float r = out_scale / sqrtf(ss / (float)N + eps);
+  const f32x4_t wv = w ? *reinterpret_cast<const f32x4_t*>(w + c0) : f32x4_t{1.f, 1.f, 1.f, 1.f};
+#pragma unroll
+  for (int e = 0; e < 4; ++e) v[e] = v[e] * r * wv[e] * gt[e];
+  T* dst = out + (size_t)t * out_ld + c0;
+  if (sizeof(T) == 2)
+    *reinterpret_cast<bf16x4_t*>(dst) = bf16x4_t{f2bits(v[0]), f2bits(v[1]), f2bits(v[2]), f2bits(v[3])};
+  else
+    *reinterpret_cast<f32x4_t*>(dst) = v;
+}
+
 // ------------------------------------------------------------------------------------------------ minGRU
 // z = sigmoid(pz + bz), u = px + bx, c = u >= 0 ? u + 1/2 : sigmoid(u); S_t = (1 - z) S_(t-1) + z c;
 // out = S_t * silu(pg).  grid (ceil(W / 256), nseq): one thread per channel walks the launch's tokens in order.
@@ -1687,6 +1730,26 @@ GRAG_API hipError_t grag_gated_rmsnorm(const float* x, const float* w, const voi
                                        int silu_gate, hipStream_t st) {
   if (T_ <= 0) return hipSuccess;
   if (groups < 1 || groups > 65535 || N % groups) return hipErrorInvalidValue;
+  const int n = N / groups;
+  const uintptr_t am = dt == 0 ? 7 : 15;
+  if (groups > 1 && n <= 256 && n % 4 == 0 && ld % 4 == 0 && goff % 4 == 0 && out_ld % 4 == 0 &&
+      ((reinterpret_cast<uintptr_t>(x) | reinterpret_cast<uintptr_t>(w)) & 15) == 0 &&
+      ((reinterpret_cast<uintptr_t>(proj) | reinterpret_cast<uintptr_t>(out)) & am) == 0) {
+#define GATED_VEC(LG)                                                                                                  \
+  hipLaunchKernelGGL((gated_rmsnorm_vec_kernel<T, LG>), dim3((unsigned)(((size_t)T_ * groups * LG + 255) / 256)), dim3(256), \
+                     0, st, x, w, (const T*)proj, ld, goff, (T*)out, out_ld, T_, n, groups, eps, out_scale, silu_gate)
+    DT_DISPATCH(dt, {
+      if (n <= 64) {
+        GATED_VEC(16);
+      } else if (n <= 128) {
+        GATED_VEC(32);
+      } else {
+        GATED_VEC(64);
+      }
+    })
+#undef GATED_VEC
+    return hipGetLastError();
+  }
   if (groups > 1 && N / groups <= 512) {
     DT_DISPATCH(dt, hipLaunchKernelGGL(gated_rmsnorm_wave_kernel<T>, dim3(T_, (groups + 3) / 4), dim3(256), 0, st, x, w,
                                        (const T*)proj, ld, goff, (T*)out, out_ld, N / groups, groups, eps, out_scale,

@@ -1,4 +1,4 @@
-"""``bench.py --hybrid [zofesun|namudra|leripel|pubulix|vudivik]``: prefill and decode throughput of a hybrid decoder beside the decoders of
+"""``bench.py --hybrid [zofesun|namudra|leripel|pubulix|vudivik|kapanex]``: prefill and decode throughput of a hybrid decoder beside the decoders of
 equal size that the engine already serves (same width, heads, head size, FFN width, layer count, vocabulary; random
 weights, synthetic token ids), all through LLMEngine.generate, and a per-kernel table: each new kernel and the
 like kernel of the closest model as a fraction of the roofline of what bounds it (HBM bytes or matrix / vector
@@ -8,7 +8,9 @@ kernel family, a layer list that is data) and Qwen2; Pubulix beside Leripel (the
 with a window instead of blocks, experts on the same grouped GEMM, the same convolution and boundary kernels) and
 Qwen2, with Namudra's latent attention as the like kernel of its latent layers; Vudivik beside Leripel (the closest: a
 state-space scan behind the same convolution, routed experts on the same grouped GEMM, the same attention kernels) and
-Qwen2, with Pubulix's window attention as the like kernel of its own."""
+Qwen2, with Pubulix's window attention as the like kernel of its own; Kapanex beside Leripel (the closest: one scan, one
+attention layer in turn, side-by-side sublayers, grouped experts with a gated shared one) and Qwen2, with Pubulix's window
+attention and Vudivik's normed rotary store as the like kernels of its own."""
 from __future__ import annotations
 
 import json
@@ -757,6 +759,153 @@ def _vudivik_kernel_table(dev, H=28, G=4, D=128, W=3584, ff=18944, T=2048, B=64,
     return rows
 
 
+def _kapanex_models(name, dev):
+    """Kapanex at a bench size: delta-rule and window-attention (1024) layers in turn, every layer beside 16 experts (4 per
+    token, 2 of 4 groups open) and a shared expert whose active width together equals the dense decoders' feed-forward;
+    beside the Leripel and Qwen2 stacks."""
+    from ..models.configs import kapanex_config
+    from ..models.kapanex import KapanexModel
+
+    W, H, G, D, ff, nl, _ = SIZES[name]
+    F = (ff // 5) // 64 * 64
+    kc = kapanex_config(f"kapanex-{name}", VOCAB, W, ("da" * nl)[:nl], heads=H, kv_heads=G, dim=D, window=1024, experts=16,
+                        top=4, groups=(4, 2), ff=F, shared_ff=ff - 4 * F)
+    mk_l, _, mk_q = _leripel_models(name, dev)
+    return (lambda: KapanexModel(kc, device=dev, seed=1)), mk_l, mk_q
+
+
+def _kapanex_kernel_table(dev, H=28, G=4, D=128, W=3584, ff=18944, T=2048, B=64, ctx=2048, bs=16, win=1024, E=16, top=4):
+    """[(kernel, seconds, bound, fraction of roofline)] for Kapanex's kernels and the like kernels of Leripel (scan,
+    convolution, gated norm, boundary, router, experts), Pubulix (window attention) and Vudivik (normed rotary store).  The
+    scans are priced in fp32 vector issue slots (2 flops each) per state number and token: 2 for the scalar-decay scan, 4
+    for the delta rule (decay, S^T k, the correction, S^T q), whatever the chunked forms add."""
+    from ..ops.attention import AttnMetadata, sink_attention
+    from ..ops.elementwise import rope_table, rope_vnorm_store
+    from ..ops.moe import moe_experts, moe_route
+    from ..ops.norm import residual_layernorm, residual_rmsnorm
+    from ..ops.recurrent import causal_conv, gated_delta, gated_rmsnorm, ssm_scan
+
+    bf = torch.bfloat16
+    i32 = dict(dtype=torch.int32, device=dev)
+    rows = []
+
+    def add(name, sec, flops=0.0, bytes_=0.0, peak=MFMA_BF16):
+        t_c, t_m = flops / peak, bytes_ / HBM_BPS
+        rows.append({"kernel": name, "us": round(sec * 1e6, 1), "bound": "flops" if t_c >= t_m else "bytes",
+                     "roofline_fraction": round(max(t_c, t_m) / sec, 4)})
+
+    nb = T // bs
+    meta = AttnMetadata(q_start=torch.tensor([0, T], **i32), ctx_len=torch.tensor([T], **i32),
+                        block_tables=(torch.arange(nb, **i32) + 1).view(1, nb), slot_mapping=torch.arange(T, **i32) + bs,
+                        max_q_len=T, num_seqs=1, num_tokens=T, state_slots=torch.tensor([0], **i32))
+    m4 = AttnMetadata(q_start=torch.arange(5, **i32) * (T // 4), ctx_len=torch.full((4,), T // 4, **i32),
+                      block_tables=meta.block_tables.expand(4, -1), slot_mapping=meta.slot_mapping, max_q_len=T // 4,
+                      num_seqs=4, num_tokens=T, state_slots=torch.arange(4, **i32))
+    nbd = ctx // bs
+    dmeta = AttnMetadata(q_start=torch.arange(B + 1, **i32), ctx_len=torch.full((B,), ctx, **i32),
+                         block_tables=(torch.arange(B * nbd, **i32) + 1).view(B, nbd), slot_mapping=None, max_q_len=1,
+                         num_seqs=B, num_tokens=B, is_decode=True, state_slots=torch.arange(B, **i32))
+    # ---- delta rule and gated norm | leripel's scan, gated norm
+    vv, C = H * D, 2 * G * D + H * D
+    ld = C + vv + 2 * H
+    pj = torch.randn(T, ld, device=dev).to(bf)
+    cw = torch.randn(C, 4, device=dev) * 0.5
+    cst = torch.zeros(B + 1, 3, C, device=dev, dtype=bf)
+    sst = torch.zeros(B + 1, H, D, D, device=dev)
+    alog, dtb, wn = torch.full((H,), -1.0, device=dev), torch.full((H,), -2.0, device=dev), torch.ones(vv, device=dev)
+    xc = causal_conv(pj, 0, cw, None, cst, meta)
+    Hs, P, N = W // 64, 64, 128
+    ch = Hs * P + 2 * N
+    pl = (torch.randn(T, 2 * Hs * P + 2 * N + Hs, device=dev) * 0.5).to(bf)
+    cwl, cbl = torch.randn(ch, 4, device=dev) * 0.5, torch.zeros(ch, device=dev)
+    cstl = torch.zeros(B + 1, 3, ch, device=dev, dtype=bf)
+    sl = torch.zeros(B + 1, Hs, N, P, device=dev)
+    z1, a1, d1 = torch.zeros(Hs, device=dev), torch.zeros(Hs, device=dev), torch.ones(Hs, device=dev)
+    xl = causal_conv(pl, Hs * P, cwl, cbl, cstl, meta)
+    outl = torch.empty(T, Hs * P, device=dev, dtype=bf)
+    wl = torch.ones(Hs * P, device=dev)
+
+    def delta(x, p, m):
+        return gated_delta(x, p, C + vv, C + vv + H, C, alog, dtb, wn, 1e-6, sst, m, H, G, D, D)
+
+    def ssm(x, p, m, out):
+        o = ssm_scan(x, p, Hs * P + ch, z1, a1, d1, sl, m, Hs, 1, N, P)
+        return gated_rmsnorm(o, wl, p, 0, 1e-6, out, gate="silu", gate_first=True)
+
+    for m, tag in ((meta, f"1 x {T}"), (m4, f"4 x {T // 4}")):
+        add(f"gated_delta prefill ({tag}, gated norm included)", _timed(lambda: delta(xc, pj, m)), flops=8.0 * T * H * D * D,
+            bytes_=T * (C + 2 * vv) * 2.0, peak=VALU_F32)
+        add(f"leripel ssm_scan + gated_rmsnorm prefill ({tag})", _timed(lambda: ssm(xl, pl, m, outl), 5, 1),
+            flops=4.0 * T * Hs * N * P, bytes_=T * (ch + 2 * Hs * P) * 2.0, peak=VALU_F32)
+    pjd, pld = pj[:B].contiguous(), pl[:B].contiguous()
+    xcd, xld = xc[:B].contiguous(), xl[:B].contiguous()
+    add("gated_delta decode (gated norm included)", _timed(lambda: delta(xcd, pjd, dmeta)), bytes_=2.0 * B * H * D * D * 4)
+    add("leripel ssm_scan + gated_rmsnorm decode", _timed(lambda: ssm(xld, pld, dmeta, outl[:B])), bytes_=2.0 * B * Hs * N * P * 4)
+    add("causal_conv prefill (4 taps)", _timed(lambda: causal_conv(pj, 0, cw, None, cst, meta)), bytes_=T * C * 2 * 2.0)
+    add("leripel causal_conv prefill (4 taps)", _timed(lambda: causal_conv(pl, Hs * P, cwl, cbl, cstl, meta)), bytes_=T * ch * 2 * 2.0)
+    add("causal_conv decode", _timed(lambda: causal_conv(pjd, 0, cw, None, cst, dmeta)), bytes_=B * C * 2 * (2 + 2 * 3.0))
+    add("leripel causal_conv decode", _timed(lambda: causal_conv(pld, Hs * P, cwl, cbl, cstl, dmeta)), bytes_=B * ch * 2 * (2 + 2 * 3.0))
+    # ---- window attention | pubulix's (window and score cap)
+    kc = torch.randn(nb + 1, G, bs, D, device=dev).to(bf)
+    vc = torch.randn(nb + 1, G, bs, D, device=dev).to(bf)
+    q = torch.randn(T, H, D, device=dev).to(bf)
+    pairs = T * (T + 1) / 2 - (T - win) * (T - win + 1) / 2
+    add(f"window attention prefill (window {win})", _timed(lambda: sink_attention(q, kc, vc, meta, 0.09, None, window=win)),
+        flops=4.0 * pairs * H * D)
+    add(f"pubulix window attention prefill (window {win})",
+        _timed(lambda: sink_attention(q, kc, vc, meta, 0.09, None, window=win, softcap=50.0)), flops=4.0 * pairs * H * D)
+    kd = torch.randn(B * nbd + 1, G, bs, D, device=dev).to(bf)
+    vd_ = torch.randn(B * nbd + 1, G, bs, D, device=dev).to(bf)
+    qd = torch.randn(B, H, D, device=dev).to(bf)
+    by = 2.0 * B * win * G * D * 2
+    add(f"window attention decode ({win} keys)", _timed(lambda: sink_attention(qd, kd, vd_, dmeta, 0.09, None, window=win)), bytes_=by)
+    add(f"pubulix window attention decode ({win} keys)",
+        _timed(lambda: sink_attention(qd, kd, vd_, dmeta, 0.09, None, window=win, softcap=50.0)), bytes_=by)
+    # ---- rotated unit heads + K/V store | the same with biases and weights
+    n = (H + 2 * G) * D
+    proj = torch.randn(T, n, device=dev).to(bf)
+    pos = torch.arange(T, **i32)
+    tab, tabh = rope_table(T, D, 1e4, dev), rope_table(T, D // 2, 1e4, dev)
+    bias, one = torch.zeros(n, device=dev), torch.ones(D, device=dev)
+    by = T * n * 2 * 2.0
+    add("rope store, unit q / k heads, half the head rotated", _timed(lambda: rope_vnorm_store(
+        proj, 0, H * D, (H + G) * D, pos, tabh, meta.slot_mapping, kc, vc, H, G, D, D, D // 2, 1e-6, vnorm=False, qw=one,
+        kw=one)), bytes_=by)
+    add("vudivik rope store with biases and head norms", _timed(lambda: rope_vnorm_store(
+        proj, 0, H * D, (H + G) * D, pos, tab, meta.slot_mapping, kc, vc, H, G, D, D, D, 1e-6, vnorm=False, bias=bias, qw=one,
+        kw=one)), bytes_=by)
+    # ---- boundary: two layer norms | one RMS norm
+    x = torch.randn(T, W, device=dev)
+    a, b = torch.randn(T, W, device=dev).to(bf), torch.randn(T, W, device=dev).to(bf)
+    e = torch.randn(T, top, W, device=dev).to(bf)
+    ec, bc, w32 = torch.rand(T, top, device=dev), torch.rand(T, device=dev), torch.ones(W, device=dev)
+    for r, tag in ((T, ""), (B, ", decode rows")):
+        xr, args = x[:r].contiguous(), [t[:r].contiguous() for t in (a, b, bc, e, ec)]
+        add(f"residual_layernorm (mixer + shared + {top} experts, two norms){tag}",
+            _timed(lambda: residual_layernorm(xr, w32, w32, 1e-6, *args)), bytes_=r * W * (8 + 2.0 * (2 + top) + 4))
+        add(f"leripel residual_rmsnorm (mixer + shared + {top} experts){tag}",
+            _timed(lambda: residual_rmsnorm(xr, *args, w32, 1e-6)), bytes_=r * W * (8 + 2.0 * (2 + top) + 2))
+    # ---- router and experts
+    F = (ff // 5) // 64 * 64
+    wr = torch.randn(E + 1, W, device=dev) * 0.05
+    sig = dict(score="sigmoid", group_top=2, scale=2.5)
+    ad = a[:B].contiguous()
+    for h, r, tag in ((a, T, "prefill"), (ad, B, "decode")):
+        add(f"moe_route {tag} (sigmoid, groups by two, {E} + 1 rows)", _timed(lambda: moe_route(h, wr, E, top, 4, 2, **sig)),
+            flops=2.0 * r * (E + 1) * W, bytes_=r * W * 2.0, peak=VALU_F32)
+        add(f"leripel moe_route {tag} (softmax, groups by one, {E} + 1 rows)", _timed(lambda: moe_route(h, wr, E, top, 4, 2)),
+            flops=2.0 * r * (E + 1) * W, bytes_=r * W * 2.0, peak=VALU_F32)
+    wgu = (torch.randn(E, 2 * F, W, device=dev) * 0.02).to(bf)
+    wd = (torch.randn(E, W, F, device=dev) * 0.02).to(bf)
+    ids, _, _ = moe_route(a, wr, E, top, 4, 2, **sig)
+    idl, _, _ = moe_route(a, wr, E, top, 4, 2)
+    for i, tag in ((ids, ""), (idl, "leripel ")):
+        add(f"{tag}experts prefill ({T} x {top} rows)", _timed(lambda: moe_experts(a, i, wgu, wd)), flops=6.0 * T * top * F * W)
+        idd = i[:B].contiguous()
+        add(f"{tag}experts decode ({B} x {top} rows)", _timed(lambda: moe_experts(ad, idd, wgu, wd)), bytes_=3.0 * E * F * W * 2)
+    return rows
+
+
 def _run_family(names, models, kernel_table) -> dict:
     """A hybrid decoder beside the decoders of equal size: ``names`` (the new one first), ``models`` (size, device) ->
     their constructors in the same order."""
@@ -783,6 +932,7 @@ FAMILIES = {
     "leripel": (("leripel", "namudra", "qwen2"), _leripel_models, _leripel_kernel_table),
     "pubulix": (("pubulix", "leripel", "qwen2"), _pubulix_models, _pubulix_kernel_table),
     "vudivik": (("vudivik", "leripel", "qwen2"), _vudivik_models, _vudivik_kernel_table),
+    "kapanex": (("kapanex", "leripel", "qwen2"), _kapanex_models, _kapanex_kernel_table),
 }
 
 
