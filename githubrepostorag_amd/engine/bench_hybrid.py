@@ -888,7 +888,7 @@ def _kapanex_kernel_table(dev, H=28, G=4, D=128, W=3584, ff=18944, T=2048, B=64,
     # ---- router and experts
     F = (ff // 5) // 64 * 64
     wr = torch.randn(E + 1, W, device=dev) * 0.05
-    sig = dict(score="sigmoid", group_top=2, scale=2.5)
+    sig = dict(score="sigmoid", group_top=2, scale=2.0)
     ad = a[:B].contiguous()
     for h, r, tag in ((a, T, "prefill"), (ad, B, "decode")):
         add(f"moe_route {tag} (sigmoid, groups by two, {E} + 1 rows)", _timed(lambda: moe_route(h, wr, E, top, 4, 2, **sig)),

@@ -50,8 +50,8 @@ def router_case(device, dtype):
     from githubrepostorag_amd.ops.moe import moe_route
 
     g = torch.Generator().manual_seed(2)
-    for E, top, groups, keep, W, T, scale in ((32, 4, 8, 4, 40, 140, 1.0), (100, 16, 4, 2, 40, 140, 1.0), (32, 3, 1, 1, 40, 9, 2.0), (6, 2, 3, 2, 40, 37, 1.7), (20, 4, 5, 3, 64, 150, 2.5), (8, 8, 1, 1, 24, 37, 1.0),
-                                              (9, 1, 9, 1, 16, 37, 0.3), (12, 3, 4, 4, 33, 131, 1.0), (24, 5, 6, 2, 264, 9, 3.0),
+    for E, top, groups, keep, W, T, scale in ((32, 4, 8, 4, 40, 140, 1.0), (100, 16, 4, 2, 40, 140, 1.0), (32, 3, 1, 1, 40, 9, 2.0), (6, 2, 3, 2, 40, 37, 1.7), (20, 4, 5, 3, 64, 150, 2.2), (8, 8, 1, 1, 24, 37, 1.0),
+                                              (9, 1, 9, 1, 16, 37, 0.3), (15, 4, 5, 5, 33, 131, 1.0), (24, 5, 6, 2, 264, 9, 3.0),
                                               (140, 6, 70, 5, 64, 20, 2.0), (1, 1, 1, 1, 24, 140, 4.0)):
         h = torch.randn(T, W, generator=g).to(dtype)
         wr = (torch.randn(E + 1, W, generator=g) * 2.0 / W ** 0.5).to(torch.bfloat16).float()
@@ -99,7 +99,7 @@ def rotary_case(device, dtype, tol):
 
 
 DELTA_SIZES = [  # H, G, d, vd, taps
-    (6, 3, 12, 20, 4), (4, 1, 64, 64, 3), (2, 2, 33, 7, 2), (3, 3, 130, 48, 1), (2, 1, 256, 256, 4), (4, 2, 128, 128, 4),
+    (6, 3, 12, 20, 4), (5, 1, 64, 96, 3), (2, 2, 33, 7, 2), (3, 3, 130, 48, 1), (2, 1, 256, 256, 4), (4, 2, 128, 128, 4),
     (1, 1, 1, 1, 2), (2, 1, 40, 255, 5),
 ]
 
